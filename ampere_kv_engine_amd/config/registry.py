@@ -12,6 +12,7 @@ import json
 import os
 from typing import Protocol
 
+from .bolatar import BolatarConfig
 from .keranex import KeranexConfig
 from .lirulix import LirulixConfig
 from .mekuvik import MekuvikConfig
@@ -69,3 +70,4 @@ register_architecture(KeranexConfig.architecture, KeranexConfig)
 register_architecture(TukevikConfig.architecture, TukevikConfig)
 register_architecture(LirulixConfig.architecture, LirulixConfig)
 register_architecture(MekuvikConfig.architecture, MekuvikConfig)
+register_architecture(BolatarConfig.architecture, BolatarConfig)

@@ -20,14 +20,21 @@ int akv_note_fed_tokens(const int* ids, const int* q_start, const int* seq_slots
 // stream [tokens, hidden] float32.  With `delta` (dtype): stream += delta / rms(delta) * post_weight (or += delta where
 // post_weight is null: stream += delta_scale * delta).  With `offset` [hidden]: stream += offset, every row, after the
 // branch.  With `out` (dtype): out = stream / rms(stream) * pre_weight, rounded once.  With `delta2` (dtype; only beside a
-// `delta` that is not normed): stream += delta_scale * (delta + delta2) - two branches that read the same input.
+// `delta` that is not normed): stream += delta_scale * (delta + delta2) - two branches that read the same input; with
+// `post_weight2` both are normed first: stream += delta_scale * (delta / rms(delta) * post_weight + delta2 / rms(delta2) *
+// post_weight2), post_eps inside both roots.
 int akv_norm_add_norm(float* stream_buf, const void* delta, const float* post_weight, float post_eps,
                       const float* pre_weight, float pre_eps, void* out, int dtype, int tokens, int hidden,
-                      float delta_scale, const float* offset, const void* delta2, hipStream_t stream);
+                      float delta_scale, const float* offset, const void* delta2, const float* post_weight2,
+                      hipStream_t stream);
 // out[n] = table[id] (with `accumulate`: out[n] += table[id]), float32; an id of -1: the token chosen last for the row's
-// request, where the slot words are given
+// request, where the slot words are given.  The row is multiplied by `scale`; with `places` [place_rows, hidden] (`dtype`) the
+// row of the token's position is added (a position beyond the table poisons the row).
 int akv_embed_rows(const int* ids, const void* table, int dtype, float* out, int tokens, int hidden, int vocab, int accumulate,
-                   const int* seq_of_token, const int* seq_slots, const int* slot_words, hipStream_t stream);
+                   const int* seq_of_token, const int* seq_slots, const int* slot_words, float scale, const void* places,
+                   int place_rows, const int* positions, hipStream_t stream);
+// values <- cap * tanh(values / cap), in place
+int akv_softcap(float* values, long count, float cap, hipStream_t stream);
 // x [tokens, width] (x_dtype: float32 or `dtype`) at x_stride per token -> out (dtype) at out_stride per token =
 // x / rms(x over the whole row) * weight (where `normed`; `weight` may be null) * act(gates[t * gate_stride + i]) * out_scale;
 // gate_act 0: no gate, 1: sigmoid, 2: silu
@@ -39,9 +46,10 @@ int akv_norm_gate_rows(const void* x, int x_dtype, long x_stride, int width, int
 int akv_embed_normed(const int* ids, const void* table, int dtype, const float* weight, float eps, float* out, int tokens,
                      int hidden, int vocab, const int* seq_of_token, const int* seq_slots, const int* slot_words,
                      hipStream_t stream);
-// out [tokens, inter] = act(gate_up[:, :inter]) * gate_up[:, inter:]; activation 0: silu, 1: the tanh form of gelu
-int akv_gated_activation(const void* gate_up, void* out, int dtype, long tokens, int inter, int activation,
-                         hipStream_t stream);
+// out [tokens, inter] = act(gate_up[:, :inter]) * gate_up[:, inter:]; activation 0: silu, 1: the tanh form of gelu; 2: with
+// g = min(gate, limit) and u = clamp(up, -limit, limit), g * sigmoid(slope g) * (u + shift)
+int akv_gated_activation(const void* gate_up, void* out, int dtype, long tokens, int inter, int activation, float limit,
+                         float slope, float shift, hipStream_t stream);
 // maps [tokens, heads, 2, vdim] -> out [tokens, heads, vdim] = (a1 - lambda[0] a2) / rms(.) * after *
 // sigmoid(gates[t * gate_stride + gate_at + h * vdim + i])
 int akv_difference_norm_gate(const void* maps, const float* lambda, float eps, float after, const void* gates,
@@ -63,11 +71,13 @@ int akv_scaled_sum(const void* a, float scale_a, const void* b, float scale_b, v
 // token's position, dimension i with i + rot_dims / 2 (`interleaved`: dimension 2 i with 2 i + 1).  `whole`: the root mean
 // square is taken over all query vectors of the token at once, and over all its key vectors.  `q_weight` [q_heads x maps x
 // dim], `k_weight` [kv_heads x maps x dim] (float32, may be null): multiplied in after the norm, before the rotation.
+// `value_eps` >= 0: value heads are divided by their root mean square (value_eps inside the root).  `temp_every` > 0: queries
+// at position p are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).
 int akv_unit_norm_write(const void* projected, long stride, int dtype, long tokens, int q_heads, int kv_heads, int dim,
                         int vdim, float eps, int normed, const int* slot_map, void* k_pages, void* v_pages, int page_size,
                         long num_pages, void* q_out, int maps, const float* table, int table_positions, int rot_dims,
                         const int* positions, const float* q_weight, const float* k_weight, int whole, int interleaved,
-                        hipStream_t stream);
+                        float value_eps, float temp_coef, int temp_every, hipStream_t stream);
 // out [tokens, q_heads, vdim].  score = (q . k) * scale, then softcap * tanh(score / softcap) where softcap > 0; a query at
 // position p sees the keys j <= p with j > p - window (window > 0; the request's first `keep_first` keys stay visible
 // behind the window) and floor(j / chunk) = floor(p / chunk) (chunk > 0);
@@ -76,12 +86,14 @@ int akv_unit_norm_write(const void* projected, long stride, int dtype, long toke
 // `row_waves` (1 .. 16) waves share a token's head: each takes every row_waves-th tile of 64 keys.  `sink_logits` [q_heads]
 // float32 (with `sink`): the extra term is exp(sink_logits[h]).  `maps` > 1: `q_heads` counts query vectors, `maps` a head
 // (out [tokens, q_heads, vdim] accordingly); vector v reads vector v % maps of its key head's record and the head's values.
+// `distance_bias` [2, q_heads] float32 (may be null): score -= bias[0, h] * ln(1 + bias[1, h] * (p - j)), after the softcap.
 int akv_gated_attention_rows(const void* q, const void* k_pages, const void* v_pages, const void* gates, long gate_stride,
                              int gate_at, const int* seq_of_token, const int* positions, const int* block_table,
                              const int* table_rows, int table_width, void* out, int dtype, long tokens, int q_heads,
                              int kv_heads, int dim, int vdim, int page_size, long num_pages, float scale, float softcap,
                              int chunk, int window, int sink, long out_stride, float out_scale, int row_waves,
-                             const float* sink_logits, int maps, int keep_first, hipStream_t stream);
+                             const float* sink_logits, int maps, int keep_first, const float* distance_bias,
+                             hipStream_t stream);
 
 // The same for rows first_row .. tokens - 1 of a bfloat16 step, on the matrix cores: keys and values 32, 64, 128 or 256
 // wide, pages of a multiple of 16 tokens (-2 otherwise); a request's rows follow each other in the order of their positions.
@@ -90,7 +102,8 @@ int akv_gated_attention_tiles(const void* q, const void* k_pages, const void* v_
                               const int* block_table, const int* table_rows, int table_width, void* out, int first_row,
                               int tokens, int q_heads, int kv_heads, int dim, int vdim, int page_size, long num_pages,
                               float scale, float softcap, int chunk, int window, int sink, long out_stride, float out_scale,
-                              const float* sink_logits, int maps, int keep_first, hipStream_t stream);
+                              const float* sink_logits, int maps, int keep_first, const float* distance_bias,
+                              hipStream_t stream);
 
 // ---- mixers with a state of fixed size (recurrent_mixers.hip) ----------------------------------------------------------
 // projected [tokens, stride]: rows [q | k (heads x dim each) | v | g (heads x vdim each)].  q and k are rotated over their
@@ -120,20 +133,52 @@ int akv_gated_linear_scan(const void* u, int dtype, const float* gates, const fl
                           const void* y, long y_stride, int seqs, int channels, int blocks, int runs, float* state,
                           long state_stride, const int* q_start, const int* seq_slots, void* out, hipStream_t stream);
 
-// ---- the gated delta rule with a decay per key channel (delta_rule.hip) ---------------------------------------------------
+// ---- the gated delta rule (delta_rule.hip) ----------------------------------------------------------------------------
 // conv [tokens, conv_stride]: rows [q (groups x dim) | k (groups x dim) | v (heads x vdim)] after their convolutions and
 // activations; head h reads q / k number h / (heads / groups).  q, k -> unit vectors (x / sqrt(sum x^2 + unit_eps)), q times
 // q_scale; beta = sigmoid(beta_logits[t * beta_stride + h]); g = exp(-rate[h] * softplus(decay_logits[t, h, d] +
-// decay_bias[h, d])).  Per request and head, S [dim, vdim] (in the slot as [heads, vdim, dim] float32):
-// S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.  out [tokens, heads x vdim] = o / rms(o) * norm_weight[i] *
-// sigmoid(gates[t, h, i]).  `workspace`: akv_delta_rule_workspace(...) floats.  `longest`: the most
-// tokens a request brings (chooses the walk's tile; the sums are the same either way).
-long akv_delta_rule_workspace(int tokens, int heads, int groups, int dim, int vdim);
+// decay_bias[h, d])) - or, `decay_per_head`, exp(-rate[h] * softplus(decay_logits[t * decay_stride + h] + decay_bias[h])).
+// Per request and head, S [dim, vdim] (in the slot as [heads, vdim, dim] float32): S <- g S; u = beta (v - S^T k);
+// S <- S + k u^T; o = S^T q.  out [tokens, heads x vdim] = o / rms(o) * norm_weight[i] * act(gates[t * gate_stride + h * vdim
+// + i]), gate_act 1: sigmoid, 2: silu.  Decay logits and gates are float32 where decays are per channel, else of `dtype`.
+// `workspace`: akv_delta_rule_workspace(...) floats.  `longest`: the most tokens a request brings (chooses the walk's tile;
+// the sums are the same either way).
+long akv_delta_rule_workspace(int tokens, int heads, int groups, int dim, int vdim, int decay_per_head);
 int akv_delta_rule(const void* conv, long conv_stride, int dtype, const void* beta_logits, long beta_stride,
-                   const float* decay_logits, const float* decay_bias, const float* rate, const float* gates,
+                   const void* decay_logits, int decay_dtype, long decay_stride, const float* decay_bias, const float* rate,
+                   int decay_per_head, const void* gates, int gate_dtype, long gate_stride, int gate_act,
                    const float* norm_weight, float unit_eps, float norm_eps, float q_scale, float* state, long state_stride,
                    const int* q_start, const int* seq_slots, float* workspace, void* out, int tokens, int seqs, int heads,
                    int groups, int dim, int vdim, int longest, hipStream_t stream);
+
+// ---- time mixing and the matrix memory (linear_states.hip) ---------------------------------------------------------------
+// out [count, tokens, width] = x_t + (x_(t-1) - x_t) * mu[s]; the row before a portion's first token lies in the request's slot
+// from element kept_at on
+int akv_token_shift(const void* x, int dtype, const float* mu, int count, const float* state, long state_stride, long kept_at,
+                    const int* seq_of_token, const int* q_start, const int* seq_slots, void* out, int tokens, int width,
+                    hipStream_t stream);
+int akv_tanh_rows(const float* x, void* out, int dtype, long count, hipStream_t stream);
+// r, k, v, gates [tokens, heads x dim] at `row_stride` per token; w = exp(-exp(decay_logits + decay_bias)) [tokens, heads x dim];
+// per request and head, S [dim, dim] (in the slot as [heads, value, key] float32): o = S^T r + (r . (bonus k)) v;
+// S <- diag(w) S + k v^T.  out = o / rms(o) * norm_weight[h, i] * silu(gate).  The slot then keeps x's last row of every request
+// (for akv_token_shift) from element kept_at on.
+long akv_time_mixing_workspace(int tokens, int heads, int dim);
+int akv_time_mixing(const void* r, const void* k, const void* v, const void* gates, int dtype, long row_stride,
+                    const float* decay_logits, const float* decay_bias, const float* bonus, const float* norm_weight, float eps,
+                    const void* x, int width, float* state, long state_stride, long kept_at, const int* q_start,
+                    const int* seq_slots, float* workspace, void* out, int tokens, int seqs, int heads, int dim, int longest,
+                    hipStream_t stream);
+// q, k [tokens, heads x dim], v and gates [tokens, heads x vdim], gate logits [tokens, heads], all at `row_stride` per token; q
+// times q_scale; i = cap tanh((i_logits + i_bias) / cap), f = logsigmoid(cap tanh((f_logits + f_bias) / cap)); m' = max(f + m, i);
+// S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone; o = S^T q / (max(|n . q|, exp(-m')) + read_eps);
+// out = o / rms(o) * norm_weight[h, i] * sigmoid(gate).  In the slot: [heads, vdim + 1, dim] (a head's last row: n), the
+// heads' m from element top_at on.
+long akv_matrix_memory_workspace(int tokens, int heads, int dim, int vdim);
+int akv_matrix_memory(const void* q, const void* k, const void* v, const void* gates, const void* i_logits, const void* f_logits,
+                      int dtype, long row_stride, const float* i_bias, const float* f_bias, float cap, float q_scale,
+                      float read_eps, const float* norm_weight, float eps, float* state, long state_stride, long top_at,
+                      const int* q_start, const int* seq_slots, float* workspace, void* out, int tokens, int seqs, int heads,
+                      int dim, int vdim, int longest, hipStream_t stream);
 
 // ---- attention over a compressed latent (latent_attention.hip) ------------------------------------------------------
 // down [tokens, q_rank (+ kv_rank + rot)]: q latent normed into `cq`; with `records`: the kv latent normed and the

@@ -25,8 +25,8 @@ LIBRARY = "libakv_kernels.so"
 # a second library, compiled when a model first needs it: token-wise kernels, mixers and the routed feed-forward of
 # designs whose norms and residual sum are float32 throughout
 PARTS_SOURCES = ("tokenwise_f32.hip", "latent_attention.hip", "selective_scan.hip", "routed.hip", "gated_attention.hip",
-                 "recurrent_mixers.hip", "delta_rule.hip")
-PARTS_HEADERS = ("common.h", "api_parts.h")
+                 "recurrent_mixers.hip", "delta_rule.hip", "linear_states.hip")
+PARTS_HEADERS = ("common.h", "api_parts.h", "state_walk.h")
 PARTS_LIBRARY = "libakv_parts.so"
 ATTENTION_SOURCE = "attention_mfma.hip"        # compiled once per head size, into its own small library
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 128, 192, 256)

@@ -1,6 +1,7 @@
 // Grouped-query attention for designs whose scores and weights are float32 and whose keys and values may differ in
 // width: unit norm of queries and keys with the cache write, and the attention itself with an optional softcap on the
-// scores, chunks of positions, a window, a sink in the softmax's denominator and a gate per head.
+// scores, a bias that grows with the distance, chunks of positions, a window, a sink in the softmax's denominator and a gate
+// per head.
 //
 // Keys lie [pages, kv_heads, page, dim], values [pages, kv_heads, vdim, page].  `gated_attention_rows` is the plain path:
 // one wave per (token, query head); keys are visited in tiles of 64 aligned to absolute key positions, so the order of
@@ -28,7 +29,9 @@ __device__ __forceinline__ void wave_sync_lds() {
 // dimensions are rotated by the token's position, dimension i with i + rot_dims / 2 - or, with `interleaved`, dimension 2 i
 // with 2 i + 1.  With `whole` the root mean square is taken over all of the token's query vectors at once (and over all of
 // its key vectors): every wave sums its side's whole projection for itself.  `q_weight` [q vectors x dim] and `k_weight`
-// [k vectors x dim] (float32, either may be null) multiply the normed values, before the rotation.
+// [k vectors x dim] (float32, either may be null) multiply the normed values, before the rotation.  With `temp_every` > 0 a
+// query is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at its position p; with `value_eps` >= 0 a value
+// head is divided by its root mean square (value_eps inside the root) before it is written.
 // One (token, item): `which` < q_vectors is a query vector, then the key vectors, then the value heads.  `given` > 0: the
 // factor 1 / rms of the item's side, formed by the caller over the whole projection; else the vector norms itself.
 template <typename T>
@@ -38,7 +41,8 @@ __device__ __forceinline__ void unit_norm_item(const T* __restrict__ row, long n
                                                int page_size, long num_pages, T* __restrict__ q_out, int maps,
                                                const float* __restrict__ table, int table_positions, int rot_dims,
                                                const int* __restrict__ positions, const float* __restrict__ q_weight,
-                                               const float* __restrict__ k_weight, int interleaved) {
+                                               const float* __restrict__ k_weight, int interleaved, float value_eps,
+                                               float temp_coef, int temp_every) {
   const int q_vectors = q_heads * maps, k_vectors = kv_heads * maps;
   if (which < q_vectors + k_vectors) {
     const bool is_q = which < q_vectors;
@@ -65,6 +69,8 @@ __device__ __forceinline__ void unit_norm_item(const T* __restrict__ row, long n
       }
       scale = rsqrtf(wave_sum(squares) / static_cast<float>(dim) + eps);
     }
+    // a temperature on queries that grows with their position
+    if (is_q && temp_every > 0) scale *= 1.f + temp_coef * logf(static_cast<float>((positions[n] + 1) / temp_every + 1));
     const float* gain = is_q ? q_weight : k_weight;
     if (gain != nullptr) gain += static_cast<long>(is_q ? which : which - q_vectors) * dim;
     if (table == nullptr || rot_dims <= 0) {
@@ -96,6 +102,16 @@ __device__ __forceinline__ void unit_norm_item(const T* __restrict__ row, long n
     if (slot < 0 || page >= num_pages) return;
     const T* x = row + static_cast<long>(q_vectors + k_vectors) * dim + static_cast<long>(h) * vdim;
     T* y = v_pages + (page * kv_heads + h) * vdim * page_size + slot % page_size;
+    if (value_eps >= 0.f) {      // values divided by their root mean square per head
+      float squares = 0.f;
+      for (int i = lane; i < vdim; i += kWave) {
+        const float v = to_float(x[i]);
+        squares += v * v;
+      }
+      const float scale = rsqrtf(wave_sum(squares) / static_cast<float>(vdim) + value_eps);
+      for (int i = lane; i < vdim; i += kWave) y[static_cast<long>(i) * page_size] = from_float<T>(to_float(x[i]) * scale);
+      return;
+    }
     for (int i = lane; i < vdim; i += kWave) y[static_cast<long>(i) * page_size] = x[i];
   }
 }
@@ -109,7 +125,8 @@ __global__ __launch_bounds__(256) void unit_norm_write_kernel(const T* __restric
                                                               const float* __restrict__ table, int table_positions,
                                                               int rot_dims, const int* __restrict__ positions,
                                                               const float* __restrict__ q_weight,
-                                                              const float* __restrict__ k_weight, int interleaved) {
+                                                              const float* __restrict__ k_weight, int interleaved,
+                                                              float value_eps, float temp_coef, int temp_every) {
   const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   const int items = (q_heads + kv_heads) * maps + kv_heads;
   const long item = static_cast<long>(blockIdx.x) * waves + wave;
@@ -117,7 +134,7 @@ __global__ __launch_bounds__(256) void unit_norm_write_kernel(const T* __restric
   const long n = item / items;
   unit_norm_item<T>(projected + n * stride, n, static_cast<int>(item % items), lane, q_heads, kv_heads, dim, vdim, eps, normed,
                     0.f, slot_map, k_pages, v_pages, page_size, num_pages, q_out, maps, table, table_positions, rot_dims,
-                    positions, q_weight, k_weight, interleaved);
+                    positions, q_weight, k_weight, interleaved, value_eps, temp_coef, temp_every);
 }
 
 // The same with the root mean square taken over all of a token's query vectors at once, and over all its key vectors: a
@@ -131,7 +148,8 @@ __global__ __launch_bounds__(1024) void unit_norm_write_whole_kernel(const T* __
                                                                     const float* __restrict__ table, int table_positions,
                                                                     int rot_dims, const int* __restrict__ positions,
                                                                     const float* __restrict__ q_weight,
-                                                                    const float* __restrict__ k_weight, int interleaved) {
+                                                                    const float* __restrict__ k_weight, int interleaved,
+                                                                    float value_eps, float temp_coef, int temp_every) {
   __shared__ float scratch[16];
   const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   const long n = blockIdx.x;
@@ -149,7 +167,7 @@ __global__ __launch_bounds__(1024) void unit_norm_write_whole_kernel(const T* __
   for (int which = wave; which < items; which += waves)
     unit_norm_item<T>(row, n, which, lane, q_heads, kv_heads, dim, vdim, eps, 1, which < q_vectors ? q_scale : k_scale, slot_map,
                       k_pages, v_pages, page_size, num_pages, q_out, maps, table, table_positions, rot_dims, positions, q_weight,
-                      k_weight, interleaved);
+                      k_weight, interleaved, value_eps, temp_coef, temp_every);
 }
 
 constexpr int kMaxValueRegs = 4;  // value widths up to 256: each lane owns dims lane, lane + 64, ...
@@ -183,7 +201,7 @@ __global__ __launch_bounds__(kMaxRowWaves * kWave) void gated_attention_rows_ker
     const int* __restrict__ block_table, const int* __restrict__ table_rows, int table_width, T* __restrict__ out,
     long tokens, int q_heads, int kv_heads, int dim, int vdim, int page_size, long num_pages, float scale, float softcap,
     int chunk, int window, int sink, long out_stride, float out_scale, const float* __restrict__ sink_logits, int maps,
-    int keep_first) {
+    int keep_first, const float* __restrict__ distance_bias) {
   // (`q_heads` counts query vectors: with `maps` > 1 a head has `maps` of them, which read the `maps` vectors of their key
   // head's record in turn and the same values; vector v's key head is still v / (q_heads / kv_heads))
   extern __shared__ unsigned char lds_raw[];
@@ -272,6 +290,8 @@ __global__ __launch_bounds__(kMaxRowWaves * kWave) void gated_attention_rows_ker
         for (int g = 0; g < G; ++g) {
           s[g] = dot[g] * scale;
           if (softcap > 0.f) s[g] = softcap * tanhf(s[g] / softcap);
+          if (distance_bias != nullptr)
+            s[g] -= distance_bias[h0 + g] * log1pf(distance_bias[q_heads + h0 + g] * static_cast<float>(pos - j));
         }
         value_at = (page * kv_heads + kvh) * vdim * page_size + j % page_size;  // values are [vdim, page_size]
       }
@@ -403,7 +423,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((DT + VT <=
     const int* __restrict__ q_start, const int* __restrict__ positions, const int* __restrict__ block_table,
     const int* __restrict__ table_rows, int table_width, bf16_t* __restrict__ out, int first_row, int tokens, int q_heads,
     int kv_heads, int page_size, long num_pages, float scale, float softcap, int chunk, int window, int sink,
-    long out_stride, float out_scale, const float* __restrict__ sink_logits, int maps, int keep_first) {
+    long out_stride, float out_scale, const float* __restrict__ sink_logits, int maps, int keep_first,
+    const float* __restrict__ distance_bias) {
   constexpr int DIM = 32 * DT, VDIM = 16 * VT;
   extern __shared__ float tile_shares[];      // [waves][2 + 4 VT][64]: what the block's waves found over their keys
   // a block is 16 rows and a head; its waves take the steps of 16 keys in turn
@@ -435,6 +456,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((DT + VT <=
   }
   float m = sink && wave == 0 ? (sink_logits != nullptr ? sink_logits[head] : 0.f) : -INFINITY, l = sink && wave == 0 ? 1.f : 0.f;
   const float inverse_cap = softcap > 0.f ? 1.f / softcap : 0.f;
+  // (the logarithm in the hardware's base)
+  const float bias_size = distance_bias != nullptr ? distance_bias[head] * 0.6931471805599453f : 0.f;
+  const float bias_rate = distance_bias != nullptr ? distance_bias[q_heads + head] : 0.f;
   float4_t o[VT];
 #pragma unroll
   for (int vt = 0; vt < VT; ++vt) o[vt] = float4_t{0.f, 0.f, 0.f, 0.f};
@@ -488,6 +512,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((DT + VT <=
             const float e = __expf(2.f * fabsf(v) * inverse_cap);
             v = copysignf(softcap * (1.f - 2.f * __frcp_rn(e + 1.f)), v);
           }
+          if (distance_bias != nullptr)      // (keys behind the query are masked below: their logarithm is taken of 1)
+            v -= bias_size * __builtin_amdgcn_logf(fmaf(bias_rate, static_cast<float>(max(my_pos - j, 0)), 1.f));
           s[i] = (in_run && (j >= my_lowest || j < keep_first) && j <= my_pos) ? v : -INFINITY;
           highest = fmaxf(highest, s[i]);
         }
@@ -589,7 +615,8 @@ int akv_gated_attention_tiles(const void* q, const void* k_pages, const void* v_
                               const int* block_table, const int* table_rows, int table_width, void* out, int first_row,
                               int tokens, int q_heads, int kv_heads, int dim, int vdim, int page_size, long num_pages,
                               float scale, float softcap, int chunk, int window, int sink, long out_stride, float out_scale,
-                              const float* sink_logits, int maps, int keep_first, hipStream_t stream) {
+                              const float* sink_logits, int maps, int keep_first, const float* distance_bias,
+                              hipStream_t stream) {
   if (tokens <= first_row) return 0;
   if (page_size % 16 != 0 || q_heads % kv_heads != 0 || maps < 1) return -2;
   const long items = static_cast<long>((tokens - first_row + 15) / 16) * q_heads;
@@ -601,7 +628,7 @@ int akv_gated_attention_tiles(const void* q, const void* k_pages, const void* v_
       static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages), static_cast<const bf16_t*>(v_pages),         \
       static_cast<const bf16_t*>(gates), gate_stride, gate_at, seq_of_token, q_start, positions, block_table, table_rows, \
       table_width, static_cast<bf16_t*>(out), first_row, tokens, q_heads, kv_heads, page_size, num_pages, scale, softcap, \
-      chunk, window, sink, out_stride, out_scale, sink_logits, maps, keep_first)
+      chunk, window, sink, out_stride, out_scale, sink_logits, maps, keep_first, distance_bias)
 #define AKV_TILES_V(DT)                    \
   switch (vdim) {                          \
     case 32: AKV_TILES(DT, 2); break;      \
@@ -626,10 +653,11 @@ int akv_unit_norm_write(const void* projected, long stride, int dtype, long toke
                         int vdim, float eps, int normed, const int* slot_map, void* k_pages, void* v_pages, int page_size,
                         long num_pages, void* q_out, int maps, const float* table, int table_positions, int rot_dims,
                         const int* positions, const float* q_weight, const float* k_weight, int whole, int interleaved,
-                        hipStream_t stream) {
+                        float value_eps, float temp_coef, int temp_every, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (q_heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || page_size <= 0 || maps < 1) return -2;
   if (table != nullptr && (rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > dim || positions == nullptr)) return -2;
+  if (temp_every > 0 && positions == nullptr) return -2;
   const long items = tokens * ((q_heads + kv_heads) * maps + kv_heads);
   if (whole && normed) {
     // (few tokens: sixteen waves a token share its items; many: four, and the tokens fill the device)
@@ -637,14 +665,15 @@ int akv_unit_norm_write(const void* projected, long stride, int dtype, long toke
     AKV_DISPATCH(dtype, T, unit_norm_write_whole_kernel<T><<<static_cast<unsigned>(tokens), threads, 0, stream>>>(
                                static_cast<const T*>(projected), stride, q_heads, kv_heads, dim, vdim, eps, slot_map,
                                static_cast<T*>(k_pages), static_cast<T*>(v_pages), page_size, num_pages, static_cast<T*>(q_out),
-                               maps, table, table_positions, rot_dims, positions, q_weight, k_weight, interleaved));
+                               maps, table, table_positions, rot_dims, positions, q_weight, k_weight, interleaved, value_eps,
+                               temp_coef, temp_every));
     return AKV_LAUNCH_STATUS();
   }
   AKV_DISPATCH(dtype, T, unit_norm_write_kernel<T><<<static_cast<unsigned>((items + 3) / 4), 256, 0, stream>>>(
                              static_cast<const T*>(projected), stride, tokens, q_heads, kv_heads, dim, vdim, eps, normed,
                              slot_map, static_cast<T*>(k_pages), static_cast<T*>(v_pages), page_size, num_pages,
                              static_cast<T*>(q_out), maps, table, table_positions, rot_dims, positions, q_weight,
-                             k_weight, interleaved));
+                             k_weight, interleaved, value_eps, temp_coef, temp_every));
   return AKV_LAUNCH_STATUS();
 }
 
@@ -653,7 +682,8 @@ int akv_gated_attention_rows(const void* q, const void* k_pages, const void* v_p
                              const int* table_rows, int table_width, void* out, int dtype, long tokens, int q_heads,
                              int kv_heads, int dim, int vdim, int page_size, long num_pages, float scale, float softcap,
                              int chunk, int window, int sink, long out_stride, float out_scale, int row_waves,
-                             const float* sink_logits, int maps, int keep_first, hipStream_t stream) {
+                             const float* sink_logits, int maps, int keep_first, const float* distance_bias,
+                             hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (maps < 1) return -2;
   const int kRowWaves = row_waves;
@@ -685,7 +715,7 @@ int akv_gated_attention_rows(const void* q, const void* k_pages, const void* v_p
                    static_cast<const T*>(q), static_cast<const T*>(k_pages), static_cast<const T*>(v_pages),            \
                    static_cast<const T*>(gates), gate_stride, gate_at, seq_of_token, positions, block_table, table_rows, \
                    table_width, static_cast<T*>(out), tokens, q_heads, kv_heads, dim, vdim, page_size, num_pages, scale, \
-                   softcap, chunk, window, sink, out_stride, out_scale, sink_logits, maps, keep_first))
+                   softcap, chunk, window, sink, out_stride, out_scale, sink_logits, maps, keep_first, distance_bias))
 #define AKV_ROWS_G(VEC)          \
   switch (bundle) {              \
     case 4: AKV_ROWS(VEC, 4); break; \

@@ -79,10 +79,11 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
                                                                  const float* __restrict__ pre_weight, float pre_eps,
                                                                  T* __restrict__ out, int hidden, float delta_scale,
                                                                  const float* __restrict__ offset,
-                                                                 const T* __restrict__ delta2) {
+                                                                 const T* __restrict__ delta2,
+                                                                 const float* __restrict__ post_weight2) {
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * hidden;
-  float4 kept[GROUPS], added[GROUPS];
+  float4 kept[GROUPS], added[GROUPS], second[GROUPS];
   // every load goes out before anything waits (a group beyond the row reads its last four values and counts for nothing)
 #pragma unroll
   for (int j = 0; j < GROUPS; ++j) {
@@ -90,13 +91,22 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
     kept[j] = read4<float>(stream + base + i);
     if (delta != nullptr) added[j] = read4<T>(delta + base + i);
     if (delta2 != nullptr) {      // a second branch beside the first: the two are added in float32 before they meet the sum
-      const float4 b = read4<T>(delta2 + base + i);
-      added[j] = make_float4(added[j].x + b.x, added[j].y + b.y, added[j].z + b.z, added[j].w + b.w);
+      second[j] = read4<T>(delta2 + base + i);
+      if (post_weight2 == nullptr)
+        added[j] = make_float4(added[j].x + second[j].x, added[j].y + second[j].y, added[j].z + second[j].z, added[j].w + second[j].w);
     }
   }
   float squares = 0.f;
   if (delta != nullptr) {
-    float post_scale = 1.f;
+    float post_scale = 1.f, second_scale = 0.f;
+    if (post_weight2 != nullptr) {      // two branches, each normed by itself
+      float acc = 0.f;
+#pragma unroll
+      for (int j = 0; j < GROUPS; ++j)
+        if ((j * 256 + static_cast<int>(threadIdx.x)) * 4 < hidden)
+          acc += second[j].x * second[j].x + second[j].y * second[j].y + second[j].z * second[j].z + second[j].w * second[j].w;
+      second_scale = delta_scale * rsqrtf(block_sum(acc, scratch) / static_cast<float>(hidden) + post_eps);
+    }
     if (post_weight != nullptr) {
       float acc = 0.f;
 #pragma unroll
@@ -104,6 +114,7 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
         if ((j * 256 + static_cast<int>(threadIdx.x)) * 4 < hidden)
           acc += added[j].x * added[j].x + added[j].y * added[j].y + added[j].z * added[j].z + added[j].w * added[j].w;
       post_scale = rsqrtf(block_sum(acc, scratch) / static_cast<float>(hidden) + post_eps);
+      if (post_weight2 != nullptr) post_scale *= delta_scale;
     }
 #pragma unroll
     for (int j = 0; j < GROUPS; ++j) {
@@ -113,6 +124,11 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
       if (post_weight != nullptr) {
         const float4 w = read4<float>(post_weight + i);
         d = make_float4(d.x * post_scale * w.x, d.y * post_scale * w.y, d.z * post_scale * w.z, d.w * post_scale * w.w);
+        if (post_weight2 != nullptr) {
+          const float4 w2 = read4<float>(post_weight2 + i), b = second[j];
+          d = make_float4(d.x + b.x * second_scale * w2.x, d.y + b.y * second_scale * w2.y, d.z + b.z * second_scale * w2.z,
+                          d.w + b.w * second_scale * w2.w);
+        }
       } else {
         d = make_float4(d.x * delta_scale, d.y * delta_scale, d.z * delta_scale, d.w * delta_scale);
       }
@@ -151,7 +167,8 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(float* __restrict__ 
                                                             const float* __restrict__ pre_weight, float pre_eps,
                                                             T* __restrict__ out, int hidden, float delta_scale,
                                                             const float* __restrict__ offset,
-                                                            const T* __restrict__ delta2) {
+                                                            const T* __restrict__ delta2,
+                                                            const float* __restrict__ post_weight2) {
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * hidden;
   float* s = stream + base;
@@ -169,6 +186,17 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(float* __restrict__ 
         }
         post_scale = rsqrtf(block_sum(acc, scratch) / static_cast<float>(hidden) + post_eps);
       }
+      if (post_weight2 != nullptr) {      // two branches, each normed by itself
+        float acc = 0.f;
+        for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+          const float v = to_float(delta2[base + i]);
+          acc += v * v;
+        }
+        const float second_scale = rsqrtf(block_sum(acc, scratch) / static_cast<float>(hidden) + post_eps);
+        for (int i = threadIdx.x; i < hidden; i += blockDim.x)
+          s[i] += delta_scale * (to_float(d[i]) * post_scale * post_weight[i] +
+                                 to_float(delta2[base + i]) * second_scale * post_weight2[i]);
+      } else
       for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
         const float both = delta2 != nullptr ? to_float(d[i]) + to_float(delta2[base + i]) : to_float(d[i]);
         s[i] += post_weight != nullptr ? both * post_scale * post_weight[i] : both * delta_scale;
@@ -221,25 +249,63 @@ __global__ __launch_bounds__(256) void embed_normed_kernel(const int* __restrict
 }
 
 // ---- rows of an embedding table into (or onto) the residual sum --------------------------------------------------------
-// out[n] = table[id] (or out[n] += table[id] with `accumulate`), float32; an id of -1 is the token chosen last for the row's
-// request, where the slot words are given.
-template <typename T>
+// out[n] = table[id] * scale (+ places[position], a table of learned position vectors), or out[n] += the same with `accumulate`;
+// float32.  An id of -1 is the token chosen last for the row's request, where the slot words are given.  A thread takes VEC
+// neighbouring columns.
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const int* __restrict__ ids, const T* __restrict__ table,
                                                          float* __restrict__ out, int hidden, int vocab, int accumulate,
                                                          const int* __restrict__ seq_of_token,
                                                          const int* __restrict__ seq_slots,
-                                                         const int* __restrict__ slot_words) {
+                                                         const int* __restrict__ slot_words, float scale,
+                                                         const T* __restrict__ places, int place_rows,
+                                                         const int* __restrict__ positions) {
   const int n = blockIdx.x;
   int id = ids[n];
   if (id == -1 && slot_words != nullptr)
     id = slot_words[static_cast<long>(seq_slots[seq_of_token[n]]) * kSlotWords + kSlotLastToken];
   float* dst = out + static_cast<size_t>(n) * hidden;
-  if (id < 0 || id >= vocab) {     // never read outside the table; a poisoned row shows the fault downstream
+  const int place = places != nullptr ? positions[n] : 0;
+  if (id < 0 || id >= vocab || (places != nullptr && (place < 0 || place >= place_rows))) {
+    // never read outside a table; a poisoned row shows the fault downstream
     for (int d = threadIdx.x; d < hidden; d += blockDim.x) dst[d] = __uint_as_float(kPoison);
     return;
   }
   const T* row = table + static_cast<size_t>(id) * hidden;
-  for (int d = threadIdx.x; d < hidden; d += blockDim.x) dst[d] = accumulate ? dst[d] + to_float(row[d]) : to_float(row[d]);
+  const T* at = places != nullptr ? places + static_cast<size_t>(place) * hidden : nullptr;
+  if constexpr (VEC == 4) {
+    for (int d = threadIdx.x * 4; d < hidden; d += blockDim.x * 4) {
+      float4 v = read4<T>(row + d);
+      v = make_float4(v.x * scale, v.y * scale, v.z * scale, v.w * scale);
+      if (at != nullptr) {
+        const float4 p = read4<T>(at + d);
+        v = make_float4(v.x + p.x, v.y + p.y, v.z + p.z, v.w + p.w);
+      }
+      if (accumulate) {
+        const float4 p = read4<float>(dst + d);
+        v = make_float4(v.x + p.x, v.y + p.y, v.z + p.z, v.w + p.w);
+      }
+      write4<float>(dst + d, v);
+    }
+  } else {
+    for (int d = threadIdx.x; d < hidden; d += blockDim.x) {
+      float v = to_float(row[d]) * scale;
+      if (at != nullptr) v += to_float(at[d]);
+      dst[d] = accumulate ? dst[d] + v : v;
+    }
+  }
+}
+
+// ---- values <- cap * tanh(values / cap) -------------------------------------------------------------------------------------
+__global__ void softcap_kernel(float* __restrict__ values, long count, float cap) {
+  const long i = (static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x) * 4;
+  if (i + 4 <= count) {
+    float4 v = read4<float>(values + i);
+    v = make_float4(cap * tanhf(v.x / cap), cap * tanhf(v.y / cap), cap * tanhf(v.z / cap), cap * tanhf(v.w / cap));
+    write4<float>(values + i, v);
+  } else {
+    for (long j = i; j < count; ++j) values[j] = cap * tanhf(values[j] / cap);
+  }
 }
 
 // ---- a row's norm, weight and gate in one pass ------------------------------------------------------------------------------
@@ -319,16 +385,41 @@ __device__ __forceinline__ float gelu_tanh_of(float z) {
   return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
+// activation 0: silu(gate) * up; 1: gelu_tanh(gate) * up; 2: with g = min(gate, limit) and u = clamp(up, -limit, limit),
+// g * sigmoid(slope g) * (u + shift)
+__device__ __forceinline__ float gated_value(float gate, float up, int activation, float limit, float slope, float shift) {
+  if (activation == 1) return gelu_tanh_of(gate) * up;
+  if (activation == 2) {
+    gate = fminf(gate, limit);
+    up = fminf(fmaxf(up, -limit), limit) + shift;
+    return gate / (1.f + expf(-slope * gate)) * up;
+  }
+  return gate / (1.f + expf(-gate)) * up;
+}
+
 template <typename T>
 __global__ void gated_activation_kernel(const T* __restrict__ gate_up, T* __restrict__ out, long tokens, int inter,
-                                        int activation) {
+                                        int activation, float limit, float slope, float shift) {
   const long index = static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (index >= tokens * inter) return;
   const long n = index / inter;
   const int i = static_cast<int>(index % inter);
   const float gate = to_float(gate_up[n * 2 * inter + i]), up = to_float(gate_up[n * 2 * inter + inter + i]);
-  const float act = activation == 1 ? gelu_tanh_of(gate) : gate / (1.f + expf(-gate));
-  out[index] = from_float<T>(act * up);
+  out[index] = from_float<T>(gated_value(gate, up, activation, limit, slope, shift));
+}
+
+// The same for widths that are a multiple of four: a thread takes four neighbouring values, a block's second index is the token.
+template <typename T>
+__global__ __launch_bounds__(256) void gated_activation4_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter,
+                                                                int activation, float limit, float slope, float shift) {
+  const long n = blockIdx.y;
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
+  if (i >= inter) return;
+  const float4 g = read4<T>(gate_up + n * 2 * inter + i), u = read4<T>(gate_up + n * 2 * inter + inter + i);
+  write4<T>(out + n * inter + i, make_float4(gated_value(g.x, u.x, activation, limit, slope, shift),
+                                             gated_value(g.y, u.y, activation, limit, slope, shift),
+                                             gated_value(g.z, u.z, activation, limit, slope, shift),
+                                             gated_value(g.w, u.w, activation, limit, slope, shift)));
 }
 
 // ---- the difference of two attention maps, normed and gated ------------------------------------------------------------
@@ -389,13 +480,19 @@ int akv_embed_normed(const int* ids, const void* table, int dtype, const float* 
   return AKV_LAUNCH_STATUS();
 }
 
-int akv_gated_activation(const void* gate_up, void* out, int dtype, long tokens, int inter, int activation,
-                         hipStream_t stream) {
+int akv_gated_activation(const void* gate_up, void* out, int dtype, long tokens, int inter, int activation, float limit,
+                         float slope, float shift, hipStream_t stream) {
   if (tokens <= 0 || inter <= 0) return 0;
-  if (activation != 0 && activation != 1) return -2;
+  if (activation < 0 || activation > 2) return -2;
+  if (inter % 4 == 0 && tokens < 65536 && reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0) {
+    const dim3 grid((inter / 4 + 255) / 256, static_cast<unsigned>(tokens));
+    AKV_DISPATCH(dtype, T, gated_activation4_kernel<T><<<grid, 256, 0, stream>>>(
+                               static_cast<const T*>(gate_up), static_cast<T*>(out), inter, activation, limit, slope, shift));
+    return AKV_LAUNCH_STATUS();
+  }
   const long count = tokens * inter;
   AKV_DISPATCH(dtype, T, gated_activation_kernel<T><<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(
-                             static_cast<const T*>(gate_up), static_cast<T*>(out), tokens, inter, activation));
+                             static_cast<const T*>(gate_up), static_cast<T*>(out), tokens, inter, activation, limit, slope, shift));
   return AKV_LAUNCH_STATUS();
 }
 
@@ -411,11 +508,27 @@ int akv_difference_norm_gate(const void* maps, const float* lambda, float eps, f
 }
 
 int akv_embed_rows(const int* ids, const void* table, int dtype, float* out, int tokens, int hidden, int vocab, int accumulate,
-                   const int* seq_of_token, const int* seq_slots, const int* slot_words, hipStream_t stream) {
+                   const int* seq_of_token, const int* seq_slots, const int* slot_words, float scale, const void* places,
+                   int place_rows, const int* positions, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (hidden <= 0 || vocab <= 0) return -2;
-  AKV_DISPATCH(dtype, T, embed_rows_kernel<T><<<tokens, 256, 0, stream>>>(ids, static_cast<const T*>(table), out, hidden, vocab,
-                                                                         accumulate, seq_of_token, seq_slots, slot_words));
+  if (places != nullptr && (place_rows <= 0 || positions == nullptr)) return -2;
+  const bool fours = hidden % 4 == 0 && reinterpret_cast<uintptr_t>(table) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0 &&
+                     reinterpret_cast<uintptr_t>(places) % 16 == 0;
+#define AKV_EMBED(VEC)                                                                                                        \
+  AKV_DISPATCH(dtype, T, embed_rows_kernel<T, VEC><<<tokens, 256, 0, stream>>>(                                               \
+                             ids, static_cast<const T*>(table), out, hidden, vocab, accumulate, seq_of_token, seq_slots,      \
+                             slot_words, scale, static_cast<const T*>(places), place_rows, positions))
+  if (fours) AKV_EMBED(4);
+  else AKV_EMBED(1);
+#undef AKV_EMBED
+  return AKV_LAUNCH_STATUS();
+}
+
+int akv_softcap(float* values, long count, float cap, hipStream_t stream) {
+  if (count <= 0) return 0;
+  if (!(cap > 0.f) || reinterpret_cast<uintptr_t>(values) % 16 != 0) return -2;
+  softcap_kernel<<<static_cast<unsigned>((count + 1023) / 1024), 256, 0, stream>>>(values, count, cap);
   return AKV_LAUNCH_STATUS();
 }
 
@@ -474,11 +587,13 @@ int akv_note_fed_tokens(const int* ids, const int* q_start, const int* seq_slots
 
 int akv_norm_add_norm(float* stream_buf, const void* delta, const float* post_weight, float post_eps,
                       const float* pre_weight, float pre_eps, void* out, int dtype, int tokens, int hidden,
-                      float delta_scale, const float* offset, const void* delta2, hipStream_t stream) {
+                      float delta_scale, const float* offset, const void* delta2, const float* post_weight2,
+                      hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (out != nullptr && pre_weight == nullptr) return -2;
-  if (delta2 != nullptr && (delta == nullptr || post_weight != nullptr)) return -2;
-#define AKV_NORM_ARGS stream_buf, static_cast<const T*>(delta), post_weight, post_eps, pre_weight, pre_eps, static_cast<T*>(out), hidden, delta_scale, offset, static_cast<const T*>(delta2)
+  if (delta2 != nullptr && (delta == nullptr || (post_weight != nullptr) != (post_weight2 != nullptr))) return -2;
+  if (post_weight2 != nullptr && delta2 == nullptr) return -2;
+#define AKV_NORM_ARGS stream_buf, static_cast<const T*>(delta), post_weight, post_eps, pre_weight, pre_eps, static_cast<T*>(out), hidden, delta_scale, offset, static_cast<const T*>(delta2), post_weight2
   AKV_DISPATCH(dtype, T, {
     if (hidden % 4 == 0 && hidden >= 4 && hidden <= 256 * 4 * 2) norm_add_norm_rows_kernel<T, 2><<<tokens, 256, 0, stream>>>(AKV_NORM_ARGS);
     else if (hidden % 4 == 0 && hidden <= 256 * 4 * 8) norm_add_norm_rows_kernel<T, 8><<<tokens, 256, 0, stream>>>(AKV_NORM_ARGS);

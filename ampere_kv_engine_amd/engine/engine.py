@@ -115,6 +115,12 @@ class Engine:
         if not self.loaded:
             raise RuntimeError("the engine has no weights yet")
         self._check_token_ids(entries)
+        reach = self.model.embedding.position_rows
+        if reach is not None:
+            for e in entries:
+                if e.seq.length + len(e.tokens) > reach:
+                    raise ValueError(f"request {e.seq.request_id!r} would reach {e.seq.length + len(e.tokens)} tokens; the model "
+                                     f"knows {reach} positions")
         if self._recordable:
             shape = self._recordable_shape(entries)
             if shape is not None:

@@ -111,6 +111,9 @@ class Scheduler:
         if total - 1 > self.engine.config.max_seq_len:
             raise ValueError(f"the request would reach {total - 1} cached tokens; the engine holds at most "
                              f"{self.engine.config.max_seq_len} per request")
+        reach = self.engine.model.embedding.position_rows
+        if reach is not None and total - 1 > reach:
+            raise ValueError(f"the request would reach {total - 1} tokens; the model knows {reach} positions")
         budget = self._budget(len(ids), max_new_tokens)
         for need, pool in zip(budget, self.pool_pages):
             if need > pool:

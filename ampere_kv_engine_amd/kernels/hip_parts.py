@@ -47,9 +47,11 @@ class PartsKernels:
                          "akv_parts_slot_layout", "akv_conv_taps", "akv_scaled_sum", "akv_unit_norm_write",
                          "akv_gated_attention_rows", "akv_gated_attention_tiles", "akv_retention", "akv_retention_chunked", "akv_gated_linear_scan", "akv_route_chosen",
                          "akv_gate_silu_mul", "akv_embed_normed", "akv_gated_activation", "akv_difference_norm_gate",
-                         "akv_delta_rule", "akv_embed_rows", "akv_norm_gate_rows", "akv_gate_activation"):
+                         "akv_delta_rule", "akv_embed_rows", "akv_norm_gate_rows", "akv_gate_activation", "akv_softcap",
+                         "akv_token_shift", "akv_tanh_rows", "akv_time_mixing", "akv_matrix_memory"):
                 getattr(lib, name).restype = ctypes.c_int
-            lib.akv_delta_rule_workspace.restype = ctypes.c_long
+            for name in ("akv_delta_rule_workspace", "akv_time_mixing_workspace", "akv_matrix_memory_workspace"):
+                getattr(lib, name).restype = ctypes.c_long
             layout = (ctypes.c_int * 3)()
             lib.akv_parts_slot_layout(layout)
             if tuple(layout) != (slots.SLOT_WORDS, slots.WORD_LAST_TOKEN, slots.WORD_FED_TOKEN):
@@ -104,11 +106,13 @@ class PartsKernels:
                                             self._stream()), "note_fed_tokens")
 
     def norm_add_norm(self, stream, delta, post_weight, post_eps, pre_weight, pre_eps, out, delta_scale: float = 1.0,
-                      offset=None, delta2=None) -> None:
+                      offset=None, delta2=None, post_weight2=None) -> None:
         """stream (float32) += delta / rms(delta) * post_weight (+= delta_scale * delta where `post_weight` is None; nothing
         where `delta` is None); then stream += offset (a float32 vector, the same on every row) where there is one; then,
         where `out` is given, out = stream / rms(stream) * pre_weight.  Float32 up to the one rounding of a stored result.
-        `delta2` (beside a `delta` that is not normed): a second branch, stream += delta_scale * (delta + delta2)."""
+        `delta2` (beside a `delta` that is not normed): a second branch, stream += delta_scale * (delta + delta2).  With
+        `post_weight2` both branches are normed: stream += delta_scale * (delta / rms(delta) * post_weight + delta2 /
+        rms(delta2) * post_weight2), with `post_eps` inside both roots."""
         tokens, hidden = stream.shape
         self._dense(stream, "stream", torch.float32)
         dtype = None
@@ -116,8 +120,8 @@ class PartsKernels:
             self._dense(delta, "delta", None, (tokens, hidden))
             dtype = delta.dtype
         if delta2 is not None:
-            if delta is None or post_weight is not None:
-                self._refuse("a second branch comes beside a first one that is added as it is")
+            if delta is None or (post_weight is None) != (post_weight2 is None):
+                self._refuse("a second branch comes beside a first one, and both are normed or neither")
             self._dense(delta2, "delta2", delta.dtype, (tokens, hidden))
         if out is not None:
             self._dense(out, "out", dtype, (tokens, hidden))
@@ -125,6 +129,10 @@ class PartsKernels:
             dtype = out.dtype
         if post_weight is not None:
             self._dense(post_weight, "post_weight", torch.float32, (hidden,))
+        if post_weight2 is not None:
+            if delta2 is None:
+                self._refuse("a norm for a second branch without one")
+            self._dense(post_weight2, "post_weight2", torch.float32, (hidden,))
         if offset is not None:
             self._dense(offset, "offset", torch.float32, (hidden,))
             dtype = dtype or torch.float32
@@ -133,19 +141,27 @@ class PartsKernels:
         self._check(self._parts().akv_norm_add_norm(_ptr(stream), _ptr(delta), _ptr(post_weight), ctypes.c_float(post_eps),
                                                     _ptr(pre_weight), ctypes.c_float(pre_eps), _ptr(out), _DTYPE_CODE[dtype],
                                                     tokens, hidden, ctypes.c_float(delta_scale), _ptr(offset), _ptr(delta2),
-                                                    self._stream()),
+                                                    _ptr(post_weight2), self._stream()),
                     "norm_add_norm")
 
     def embed_add(self, ids, table, out, ctx=None) -> None:
         """out[n] += table[id], float32: the embedding's rows added to a residual sum that already holds something.  With
         the step's context an id of -1 is the token chosen last for the row's request."""
+        self._embed_rows(ids, table, out, ctx, accumulate=True)
+
+    def embed_scaled(self, ids, table, scale: float, places, out, ctx) -> None:
+        """out[n] = table[id] * scale (+ places[position of the token], a table [positions, hidden], where there is one),
+        float32.  An id of -1 is the token chosen last for the row's request."""
+        self._embed_rows(ids, table, out, ctx, scale=scale, places=places)
+
+    def _embed_rows(self, ids, table, out, ctx, accumulate: bool = False, scale: float = 1.0, places=None) -> None:
         tokens = ids.shape[0]
         self._dense(ids, "ids", torch.int32, (tokens,))
         self._dense(table, "table")
         vocab, hidden = table.shape
         self._dense(out, "out", torch.float32, (tokens, hidden))
         words = getattr(ctx, "slot_words", None) if ctx is not None else None
-        seq_of_token = seq_slots = None
+        seq_of_token = seq_slots = positions = None
         if words is not None:
             seq_of_token, seq_slots = ctx.seq_of_token, ctx.seq_slots
             self._dense(words, "slot_words", torch.int32)
@@ -153,9 +169,23 @@ class PartsKernels:
             self._dense(seq_slots, "seq_slots", torch.int32, (ctx.num_seqs,))
             if max(ctx.host_seq_slots) >= words.shape[0]:
                 self._refuse("a request's slot lies outside the slot words")
+        if places is not None:
+            self._dense(places, "places", table.dtype)
+            if places.dim() != 2 or places.shape[1] != hidden:
+                self._refuse(f"position vectors must be [positions, {hidden}], got {tuple(places.shape)}")
+            positions = ctx.positions
+            self._dense(positions, "positions", torch.int32, (tokens,))
         self._check(self._parts().akv_embed_rows(_ptr(ids), _ptr(table), self._code_of(table), _ptr(out), tokens, hidden, vocab,
-                                                 1, _ptr(seq_of_token), _ptr(seq_slots), _ptr(words), self._stream()),
-                    "embed_add")
+                                                 1 if accumulate else 0, _ptr(seq_of_token), _ptr(seq_slots), _ptr(words),
+                                                 ctypes.c_float(scale), _ptr(places), places.shape[0] if places is not None else 0,
+                                                 _ptr(positions), self._stream()), "embed_rows")
+
+    def softcap(self, values, cap: float) -> None:
+        """values (float32) <- cap * tanh(values / cap), in place."""
+        self._dense(values, "values", torch.float32)
+        if cap <= 0:
+            self._refuse(f"a softcap is positive, not {cap}")
+        self._check(self._parts().akv_softcap(_ptr(values), _long(values.numel()), ctypes.c_float(cap), self._stream()), "softcap")
 
     GATE_ACTS = {None: 0, "sigmoid": 1, "silu": 2}
 
@@ -214,17 +244,20 @@ class PartsKernels:
                                                    ctypes.c_float(eps), _ptr(out), tokens, hidden, vocab, _ptr(seq_of_token),
                                                    _ptr(seq_slots), _ptr(words), self._stream()), "embed_normed")
 
-    GATED_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+    GATED_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 
-    def gated_activation(self, gate_up, out, activation: str) -> None:
-        """out [tokens, inter] = act(gate_up[:, :inter]) * gate_up[:, inter:], in float32 with one rounding."""
+    def gated_activation(self, gate_up, out, activation: str, limit: float = 0.0, slope: float = 1.0, shift: float = 0.0) -> None:
+        """out [tokens, inter] = act(gate_up[:, :inter]) * gate_up[:, inter:], in float32 with one rounding.  "clamped": with
+        g = min(gate, limit) and u = clamp(up, -limit, limit), g * sigmoid(slope * g) * (u + shift)."""
         tokens, inter = out.shape
         self._dense(out, "out")
         self._dense(gate_up, "gate_up", out.dtype, (tokens, 2 * inter))
         if activation not in self.GATED_ACTIVATIONS:
             self._refuse(f"a gated feed-forward's activation is one of {sorted(self.GATED_ACTIVATIONS)}, not {activation!r}")
         self._check(self._parts().akv_gated_activation(_ptr(gate_up), _ptr(out), self._code_of(out), _long(tokens), inter,
-                                                       self.GATED_ACTIVATIONS[activation], self._stream()), "gated_activation")
+                                                       self.GATED_ACTIVATIONS[activation], ctypes.c_float(limit),
+                                                       ctypes.c_float(slope), ctypes.c_float(shift), self._stream()),
+                    "gated_activation")
 
     def difference_norm_gate(self, maps, lam, eps: float, after: float, gates, gate_at: int, heads: int, vdim: int, out) -> None:
         """maps [tokens, heads * 2 * vdim] (per head: map 1, map 2) -> out [tokens, heads * vdim] = (a1 - lam a2) /
@@ -467,51 +500,152 @@ class PartsKernels:
                          f"{heads} / {groups} heads of {dim}")
 
     def delta_rule(self, conv, beta_logits, beta_at: int, decay_logits, decay_bias, rate, gates, norm_weight, unit_eps: float,
-                   norm_eps: float, q_scale: float, heads: int, groups: int, dim: int, vdim: int, state, ctx, out) -> None:
+                   norm_eps: float, q_scale: float, heads: int, groups: int, dim: int, vdim: int, state, ctx, out,
+                   decay_at: int | None = None, gate_at: int = 0, gate: str = "sigmoid") -> None:
         """conv [tokens, 2 * groups * dim + heads * vdim]: q, k and v after their convolutions and activations.  q and k
         become unit vectors per head (x / sqrt(sum x^2 + unit_eps); q times q_scale); beta = sigmoid(beta_logits[:, beta_at +
         h]); g = exp(-rate[h] * softplus(decay_logits[t, h, d] + decay_bias[h, d])).  Per request and head, token after
         token: S <- g S (rows are key channels); u = beta (v - S^T k); S <- S + k u^T; o = S^T q.  out [tokens, heads * vdim]
         = o / rms(o) * norm_weight * sigmoid(gates).  S lies at the start of the request's slot of `state`, float32, as
-        [heads, vdim, dim]."""
+        [heads, vdim, dim].  With `decay_at` a head has one decay, exp(-rate[h] * softplus(decay_logits[:, decay_at + h] +
+        decay_bias[h])), and the gates are columns gate_at .. of `gates` (both of conv's dtype, behind sigmoid or silu)."""
         tokens = conv.shape[0]
         width = 2 * groups * dim + heads * vdim
+        per_head = decay_at is not None
         self._dense(conv, "conv", None, (tokens, width))
         self._dense(beta_logits, "beta_logits", conv.dtype)
         if beta_logits.dim() != 2 or beta_logits.shape[0] != tokens or beta_at < 0 or beta_at + heads > beta_logits.shape[1]:
             self._refuse(f"beta_logits must be [tokens, at least {beta_at + heads}], got {tuple(beta_logits.shape)}")
-        self._dense(decay_logits, "decay_logits", torch.float32, (tokens, heads * dim))
-        self._dense(decay_bias, "decay_bias", torch.float32, (heads * dim,))
+        if per_head:
+            for what, rows, at, columns in (("decay_logits", decay_logits, decay_at, heads), ("gates", gates, gate_at, heads * vdim)):
+                self._dense(rows, what, conv.dtype)
+                if rows.dim() != 2 or rows.shape[0] != tokens or at < 0 or at + columns > rows.shape[1]:
+                    self._refuse(f"{what} must be [tokens, at least {at + columns}], got {tuple(rows.shape)}")
+            self._dense(decay_bias, "decay_bias", torch.float32, (heads,))
+        else:
+            self._dense(decay_logits, "decay_logits", torch.float32, (tokens, heads * dim))
+            self._dense(decay_bias, "decay_bias", torch.float32, (heads * dim,))
+            self._dense(gates, "gates", torch.float32, (tokens, heads * vdim))
+            decay_at = gate_at = 0
+        if gate not in ("sigmoid", "silu"):
+            self._refuse(f"the outputs' gate is 'sigmoid' or 'silu', not {gate!r}")
         self._dense(rate, "rate", torch.float32, (heads,))
-        self._dense(gates, "gates", torch.float32, (tokens, heads * vdim))
         self._dense(norm_weight, "norm_weight", torch.float32, (vdim,))
         self._dense(out, "out", conv.dtype, (tokens, heads * vdim))
-        self._dense(state, "state", torch.float32)
-        if state.dim() != 2 or state.shape[1] < heads * dim * vdim:
-            self._refuse(f"the state must be [slots, at least {heads * dim * vdim}], got {tuple(state.shape)}")
-        if max(ctx.host_seq_slots) >= state.shape[0]:
-            self._refuse("a request's slot lies outside the state")
+        self._state_of_slots(state, heads * dim * vdim, ctx)
         self.check_delta_rule_sizes(heads, groups, dim, vdim)
         self._step_arrays(ctx, tokens)
         lib = self._parts()
-        workspace = self._delta_workspace(int(lib.akv_delta_rule_workspace(tokens, heads, groups, dim, vdim)))
+        workspace = self._walk_workspace(int(lib.akv_delta_rule_workspace(tokens, heads, groups, dim, vdim, 1 if per_head else 0)))
         self._check(lib.akv_delta_rule(
             _ptr(conv), _long(width), self._code_of(conv), _ptr_at(beta_logits, beta_at), _long(beta_logits.shape[1]),
-            _ptr(decay_logits), _ptr(decay_bias), _ptr(rate), _ptr(gates), _ptr(norm_weight), ctypes.c_float(unit_eps),
+            _ptr_at(decay_logits, decay_at), self._code_of(decay_logits), _long(decay_logits.shape[1]), _ptr(decay_bias),
+            _ptr(rate), 1 if per_head else 0, _ptr_at(gates, gate_at), self._code_of(gates), _long(gates.shape[1]),
+            self.GATE_ACTS[gate], _ptr(norm_weight), ctypes.c_float(unit_eps),
             ctypes.c_float(norm_eps), ctypes.c_float(q_scale), _ptr(state), _long(state.shape[1]), _ptr(ctx.q_start),
             _ptr(ctx.seq_slots), _ptr(workspace), _ptr(out), tokens, ctx.num_seqs, heads, groups, dim, vdim,
             int(ctx.max_new_tokens) or tokens, self._stream()),
             "delta_rule")
 
-    def _delta_workspace(self, need: int) -> torch.Tensor:
-        """Where the tokens' unit vectors, decays and raw outputs lie during a step."""
-        held = self.__dict__.get("_delta_buffer")
+    def _state_of_slots(self, state, need: int, ctx) -> None:
+        self._dense(state, "state", torch.float32)
+        if state.dim() != 2 or state.shape[1] < need:
+            self._refuse(f"the state must be [slots, at least {need}], got {tuple(state.shape)}")
+        if max(ctx.host_seq_slots) >= state.shape[0]:
+            self._refuse("a request's slot lies outside the state")
+
+    def _walk_workspace(self, need: int) -> torch.Tensor:
+        """Where the tokens' vectors, decays and raw outputs lie while a matrix state walks over them."""
+        held = self.__dict__.get("_walk_buffer")
         if held is None or held.numel() < need:
             if torch.cuda.is_current_stream_capturing():
-                self._refuse("a recorded step needs more room for the delta rule's tokens than the steps before it")
-            self.__dict__.setdefault("_delta_outgrown", []).append(held)
-            held = self.__dict__["_delta_buffer"] = torch.empty(max(need, 1 << 22), dtype=torch.float32, device=self.device)
+                self._refuse("a recorded step needs more room for a recurrence's tokens than the steps before it")
+            self.__dict__.setdefault("_walk_outgrown", []).append(held)
+            held = self.__dict__["_walk_buffer"] = torch.empty(max(need, 1 << 22), dtype=torch.float32, device=self.device)
         return held
+
+    # ---- time mixing -----------------------------------------------------------------------------------------------------
+    def check_state_sizes(self, heads: int, dim: int, vdim: int) -> None:
+        if heads <= 0 or not 0 < dim <= 2048 or vdim <= 0:
+            self._refuse(f"a walked state takes keys up to 2048 wide, not {heads} heads of {dim} x {vdim}")
+
+    def token_shift(self, x, mu, state, kept_at: int, ctx, out) -> None:
+        """out [count, tokens, width] = x_t + (x_(t-1) - x_t) * mu[s] for the rows of `mu` [count, width] (float32); the row
+        before a portion's first token lies in its request's slot of `state` from element `kept_at` on."""
+        tokens, width = x.shape
+        count = mu.shape[0]
+        self._dense(x, "x")
+        self._dense(mu, "mu", torch.float32, (count, width))
+        self._dense(out, "out", x.dtype, (count, tokens, width))
+        self._state_of_slots(state, kept_at + width, ctx)
+        self._step_arrays(ctx, tokens)
+        self._check(self._parts().akv_token_shift(
+            _ptr(x), self._code_of(x), _ptr(mu), count, _ptr(state), _long(state.shape[1]), _long(kept_at),
+            _ptr(ctx.seq_of_token), _ptr(ctx.q_start), _ptr(ctx.seq_slots), _ptr(out), tokens, width, self._stream()),
+            "token_shift")
+
+    def tanh_rows(self, x, out) -> None:
+        """out = tanh(x), float32 -> out's dtype."""
+        self._dense(x, "x", torch.float32)
+        self._dense(out, "out", None, tuple(x.shape))
+        self._check(self._parts().akv_tanh_rows(_ptr(x), _ptr(out), self._code_of(out), _long(x.numel()), self._stream()), "tanh_rows")
+
+    def time_mixing(self, rkvg, decay_logits, decay_bias, bonus, norm_weight, eps: float, x, heads: int, dim: int, state,
+                    kept_at: int, ctx, out) -> None:
+        """rkvg [4, tokens, heads * dim]: r, k, v and gates; w = exp(-exp(decay_logits + decay_bias)).  Per request and head,
+        token after token: o = S^T r + (r . (bonus k)) v; S <- diag(w) S + k v^T.  out = o / rms(o) * norm_weight *
+        silu(gates).  S lies at the start of the request's slot as [heads, value, key]; afterwards the slot keeps the
+        portion's last row of `x` from element `kept_at` on (what `token_shift` reads)."""
+        tokens, width = x.shape
+        wide = heads * dim
+        self._dense(rkvg, "rkvg", None, (4, tokens, wide))
+        self._dense(decay_logits, "decay_logits", torch.float32, (tokens, wide))
+        for name, vector in (("decay_bias", decay_bias), ("bonus", bonus), ("norm_weight", norm_weight)):
+            self._dense(vector, name, torch.float32, (wide,))
+        self._dense(x, "x", rkvg.dtype)
+        self._dense(out, "out", rkvg.dtype, (tokens, wide))
+        self._state_of_slots(state, max(wide * dim, kept_at + width), ctx)
+        self.check_state_sizes(heads, dim, dim)
+        self._step_arrays(ctx, tokens)
+        lib = self._parts()
+        workspace = self._walk_workspace(int(lib.akv_time_mixing_workspace(tokens, heads, dim)))
+        r, k, v, g = (_ptr(rkvg[i]) for i in range(4))
+        self._check(lib.akv_time_mixing(
+            r, k, v, g, self._code_of(rkvg), _long(wide), _ptr(decay_logits), _ptr(decay_bias), _ptr(bonus), _ptr(norm_weight),
+            ctypes.c_float(eps), _ptr(x), width, _ptr(state), _long(state.shape[1]), _long(kept_at), _ptr(ctx.q_start),
+            _ptr(ctx.seq_slots), _ptr(workspace), _ptr(out), tokens, ctx.num_seqs, heads, dim,
+            int(ctx.max_new_tokens) or tokens, self._stream()), "time_mixing")
+
+    # ---- the matrix memory -----------------------------------------------------------------------------------------------
+    def matrix_memory(self, projected, i_bias, f_bias, cap: float, read_eps: float, norm_weight, eps: float, heads: int, dim: int,
+                      vdim: int, state, top_at: int, ctx, out) -> None:
+        """projected [tokens, q | k (heads * dim each) | v | g (heads * vdim each) | i | f (heads each)].  q times dim^(-1/2);
+        i = cap tanh((. + i_bias) / cap), f = logsigmoid(cap tanh((. + f_bias) / cap)).  Per request and head, token after
+        token: m' = max(f + m, i); S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone; o = S^T q /
+        (max(|n . q|, exp(-m')) + read_eps).  out = o / rms(o) * norm_weight * sigmoid(g).  In the slot: S and n as [heads,
+        vdim + 1, dim] (n the last row of a head), the heads' m from element `top_at` on."""
+        tokens = projected.shape[0]
+        qk, vs = heads * dim, heads * vdim
+        self._dense(projected, "projected")
+        if projected.dim() != 2 or projected.shape[1] != 2 * (qk + vs + heads):
+            self._refuse(f"projected must be [tokens, {2 * (qk + vs + heads)}], got {tuple(projected.shape)}")
+        for name, vector in (("i_bias", i_bias), ("f_bias", f_bias)):
+            self._dense(vector, name, torch.float32, (heads,))
+        self._dense(norm_weight, "norm_weight", torch.float32, (vs,))
+        self._dense(out, "out", projected.dtype, (tokens, vs))
+        self._state_of_slots(state, top_at + heads, ctx)
+        if top_at < heads * dim * (vdim + 1) or cap <= 0:
+            self._refuse("the running maxima lie behind the state, and the gates' cap is positive")
+        self.check_state_sizes(heads, dim, vdim)
+        self._step_arrays(ctx, tokens)
+        lib = self._parts()
+        workspace = self._walk_workspace(int(lib.akv_matrix_memory_workspace(tokens, heads, dim, vdim)))
+        at = [_ptr_at(projected, column) for column in (0, qk, 2 * qk, 2 * qk + vs, 2 * (qk + vs), 2 * (qk + vs) + heads)]
+        self._check(lib.akv_matrix_memory(
+            *at, self._code_of(projected), _long(projected.shape[1]), _ptr(i_bias), _ptr(f_bias), ctypes.c_float(cap),
+            ctypes.c_float(dim ** -0.5), ctypes.c_float(read_eps), _ptr(norm_weight), ctypes.c_float(eps), _ptr(state),
+            _long(state.shape[1]), _long(top_at), _ptr(ctx.q_start), _ptr(ctx.seq_slots), _ptr(workspace), _ptr(out), tokens,
+            ctx.num_seqs, heads, dim, vdim, int(ctx.max_new_tokens) or tokens, self._stream()), "matrix_memory")
 
     def selective_scan(self, x, dt, bc, xz, a, d, state, taps, ctx, out) -> None:
         """Per request and channel, token after token: S <- exp(softplus(dt) A) S + softplus(dt) x B, y = S C + D x,
@@ -624,7 +758,8 @@ class PartsKernels:
 
     def unit_norm_write(self, projected, q_heads, kv_heads, dim, vdim, eps, slot_map, k_pages, v_pages, q_out, at: int = 0,
                         maps: int = 1, table=None, rot_dims: int = 0, positions=None, q_weight=None, k_weight=None,
-                        whole: bool = False, interleaved: bool = False) -> None:
+                        whole: bool = False, interleaved: bool = False, value_eps: float | None = None,
+                        temperature: tuple | None = None) -> None:
         """projected [tokens, ... | q | k | v | ...] with q at column `at`: the query heads divided by their root mean square (eps inside the root;
         `eps` None: as they are) -> q_out; with `slot_map` the key heads, the same way, and the value heads into the
         tokens' slots of the pages.  `maps` > 1: a head's queries and keys are `maps` vectors of `dim` side by side, each
@@ -632,7 +767,9 @@ class PartsKernels:
         rot_dims / 2, 2] (cos, sin): every vector's first `rot_dims` dimensions are rotated by the token's position
         (`positions`), dimension i with i + rot_dims / 2 (`interleaved`: 2 i with 2 i + 1), after the norm.  `whole`: the
         root mean square is taken over all of a token's query vectors at once, and over all its key vectors.  `q_weight`,
-        `k_weight` (float32, one value per column of the queries and of the keys): multiplied in after the norm."""
+        `k_weight` (float32, one value per column of the queries and of the keys): multiplied in after the norm.
+        `value_eps`: every value head is divided by its root mean square (value_eps inside the root) before it is written.
+        `temperature` (coef, every): a query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)."""
         tokens = projected.shape[0]
         if q_weight is not None:
             self._dense(q_weight, "q_weight", torch.float32, (q_heads * maps * dim,))
@@ -653,23 +790,32 @@ class PartsKernels:
                              f"got {tuple(table.shape)} for {rot_dims}")
             self._dense(positions, "positions", torch.int32, (tokens,))
             table_positions = table.shape[0]
+        coef, every = (float(temperature[0]), int(temperature[1])) if temperature is not None else (0.0, 0)
+        if temperature is not None:
+            if every <= 0:
+                self._refuse(f"a temperature that grows every {every} positions")
+            self._dense(positions, "positions", torch.int32, (tokens,))
         self._check(self._parts().akv_unit_norm_write(
             _ptr_at(projected, at), _long(projected.shape[1]), self._code_of(projected), _long(tokens), q_heads, kv_heads, dim,
             vdim, ctypes.c_float(eps if eps is not None else 0.0), 0 if eps is None else 1, _ptr(slot_map), _ptr(k_pages),
             _ptr(v_pages), page_size, _long(num_pages), _ptr(q_out), maps, _ptr(table), table_positions,
-            rot_dims if table is not None else 0, _ptr(positions) if table is not None else ctypes.c_void_p(0),
-            _ptr(q_weight), _ptr(k_weight), 1 if whole else 0, 1 if interleaved else 0, self._stream()), "unit_norm_write")
+            rot_dims if table is not None else 0,
+            _ptr(positions) if table is not None or temperature is not None else ctypes.c_void_p(0),
+            _ptr(q_weight), _ptr(k_weight), 1 if whole else 0, 1 if interleaved else 0,
+            ctypes.c_float(value_eps if value_eps is not None else -1.0), ctypes.c_float(coef), every, self._stream()),
+            "unit_norm_write")
 
     def gated_attention(self, q, k_pages, v_pages, gates, gate_at, ctx, meta, q_heads, kv_heads, dim, vdim, scale, softcap,
                         chunk, window, sink, out, out_at: int = 0, out_scale: float = 1.0, sink_logits=None,
-                        maps: int = 1, keep_first: int = 0) -> None:
+                        maps: int = 1, keep_first: int = 0, distance_bias=None) -> None:
         """Every query head attends the keys of its request that it sees (see `parts/gated_attention.py`) -> columns
         out_at .. out_at + q_heads * vdim of `out`, times `out_scale`; `gates` [tokens, width]: head h's output times
         sigmoid(gates[t, gate_at + h]).  `sink_logits` [q_heads] float32 (with `sink`): the denominator's extra term is
         exp(sink_logits[h]) instead of exp(0).  `maps` > 1: a head has `maps` query vectors, each an attention of its own
         over the vector of the same number in its key head's record ([pages, kv_heads, page, maps * dim]) and over the
         head's values; out then holds q_heads * maps outputs a token, a head's maps side by side.  `keep_first`: a request's
-        first so many keys stay visible behind the window."""
+        first so many keys stay visible behind the window.  `distance_bias` [2, q_heads] float32: the score of key j for a query
+        at position p is lowered by bias[0, h] * ln(1 + bias[1, h] * (p - j)), after the softcap."""
         tokens = q.shape[0]
         heads = q_heads
         q_heads = heads * maps          # (from here on: query vectors)
@@ -684,6 +830,8 @@ class PartsKernels:
             self._dense(sink_logits, "sink_logits", torch.float32, (q_heads,))
             if not sink:
                 self._refuse("sink logits without a sink")
+        if distance_bias is not None:
+            self._dense(distance_bias, "distance_bias", torch.float32, (2, q_heads))
         gate_stride = 0
         if gates is not None:
             self._dense(gates, "gates", q.dtype)
@@ -704,7 +852,7 @@ class PartsKernels:
             self._refuse("a request is longer than its row of the block table")
         tail = (ctypes.c_float(scale), ctypes.c_float(softcap if softcap is not None else 0.0),
                 int(chunk) if chunk is not None else 0, int(window) if window is not None else 0, 1 if sink else 0,
-                _long(out.shape[1]), ctypes.c_float(out_scale), _ptr(sink_logits), maps, int(keep_first), self._stream())
+                _long(out.shape[1]), ctypes.c_float(out_scale), _ptr(sink_logits), maps, int(keep_first), _ptr(distance_bias), self._stream())
         singles = tokens
         if (q.dtype == torch.bfloat16 and dim in self.MATRIX_CORE_HEAD_DIMS and vdim in self.MATRIX_CORE_HEAD_DIMS
                 and page_size % 16 == 0 and out.shape[1] % 4 == 0 and out_at % 4 == 0):
@@ -723,8 +871,8 @@ class PartsKernels:
             self._check(self._parts().akv_gated_attention_rows(
                 _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(gates), _long(gate_stride), gate_at, _ptr(ctx.seq_of_token),
                 _ptr(ctx.positions), _ptr(meta.block_table), _ptr(meta.rows), meta.width, _ptr_at(out, out_at),
-                self._code_of(q), _long(singles), q_heads, kv_heads, dim, vdim, page_size, _long(num_pages), *tail[:-4], row_waves,
-                *tail[-4:]), "gated_attention")
+                self._code_of(q), _long(singles), q_heads, kv_heads, dim, vdim, page_size, _long(num_pages), *tail[:-5], row_waves,
+                *tail[-5:]), "gated_attention")
 
     # ---- mixers with a state of fixed size -----------------------------------------------------------------------------
     def check_retention_sizes(self, heads: int, dim: int, vdim: int) -> None:

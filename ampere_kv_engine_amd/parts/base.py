@@ -271,6 +271,24 @@ class NormedDelta(Unsettled):
         self.norm.add_normed(stream, self.delta)
 
 
+class NormedPair(Unsettled):
+    """The outputs of two mixers side by side, each of which is still to be normed over the model's width with a weight of
+    its own (float32, one rounding): stream += scale * (delta / rms(delta) * weight + second / rms(second) * second_weight).
+    What `parts/parallel.py` hands on where its block says that it takes such a thing (`ctx.takes_unsettled_branch`)."""
+
+    def __init__(self, delta: torch.Tensor, weight: torch.Tensor, second: torch.Tensor, second_weight: torch.Tensor, eps: float,
+                 scale: float, kernels):
+        self.delta, self.weight, self.second, self.second_weight = delta, weight, second, second_weight
+        self.eps, self.scale, self.kernels = float(eps), float(scale), kernels
+
+    def times(self, scale: float) -> "NormedPair":
+        return NormedPair(self.delta, self.weight, self.second, self.second_weight, self.eps, self.scale * scale, self.kernels)
+
+    def settle(self, stream: torch.Tensor) -> None:
+        self.kernels.norm_add_norm(stream, self.delta, self.weight, self.eps, None, 0.0, None, delta_scale=self.scale,
+                                   delta2=self.second, post_weight2=self.second_weight)
+
+
 class StreamSums:
     """What a branch hands on instead of its output when its last product has already added that output to the
     residual sum (`Linear.add_to_stream`): the partial sums of squares of the new residual rows, float32, from which

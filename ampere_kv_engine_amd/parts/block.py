@@ -188,7 +188,10 @@ class ScaledPreNormBlock(Part):
         ctx.fold_into_stream, ctx.fold_gain = False, None      # no branch of this block adds itself to the stream
         shape = (stream.shape[0], self.hidden)
         normed = self.norms[0].after(stream, pending, ctx.arena.take(shape, self.rt.dtype))
-        mixed = ScaledDelta(self.mixer.forward(normed, ctx, cache, writes_cache), self.scale, self.rt.kernels)
+        ctx.takes_unsettled_branch = True         # (two branches that are still to be normed may meet the stream in the next norm)
+        mixed = self.mixer.forward(normed, ctx, cache, writes_cache)
+        ctx.takes_unsettled_branch = False
+        mixed = mixed.times(self.scale) if isinstance(mixed, Unsettled) else ScaledDelta(mixed, self.scale, self.rt.kernels)
         if not self.has_feed_forward:
             return mixed
         normed = self.norms[1].after(stream, mixed, ctx.arena.take(shape, self.rt.dtype))

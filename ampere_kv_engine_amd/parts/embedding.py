@@ -11,6 +11,9 @@ from .linear import Linear
 
 
 class Embedding(Part):
+    # positions a request may reach where the embedding reads a table of them; None: no such table
+    position_rows: int | None = None
+
     def __init__(self, spec, runtime):
         self.rt = runtime
         self.vocab, self.hidden = int(spec["vocab_size"]), int(spec["hidden_size"])
@@ -62,6 +65,30 @@ class NormedEmbedding(Embedding):
         return stream
 
 
+class PositionedEmbedding(Embedding):
+    """The token's row times a constant, plus a learned vector of the token's position: x = table[id] * scale + places[p]
+    (the vector as it is), in float32 (one kernel).  `positions` names the table of vectors, `position_rows` how many it
+    holds: a request cannot grow beyond them."""
+
+    def __init__(self, spec, runtime):
+        super().__init__(spec, runtime)
+        self.scale = float(spec.get("scale", 1.0))
+        self.positions_name = spec["positions"]
+        self.position_rows = int(spec["position_rows"])
+        self.places = None
+
+    def tensors(self, prefix=""):
+        return super().tensors() + [TensorSpec(self.positions_name, (self.position_rows, self.hidden), EMBEDDING)]
+
+    def load(self, fetch, prefix=""):
+        super().load(fetch)
+        self.places = fetch(self.tensors()[1]).contiguous()
+
+    def forward(self, token_ids, stream, ctx=None):
+        self.rt.kernels.embed_scaled(token_ids, self.weight, self.scale, self.places, stream, ctx)
+        return stream
+
+
 class RowTable(Part):
     """A table [rows, hidden] of vectors, float32, of which the model's pass adds one to every token's residual sum
     where the run order says so (`RunEntry.adds_row`)."""
@@ -110,7 +137,7 @@ class PairHashEmbedding(Embedding):
 
 
 class LinearHead(Part):
-    """logits = x W^T in float32.  When `tied_to` names the embedding, the head uses that matrix and the
+    """logits = x W^T in float32; with `softcap` c, logits <- c * tanh(logits / c).  When `tied_to` names the embedding, the head uses that matrix and the
     file may leave the head's own tensor out."""
 
     def __init__(self, spec, runtime):
@@ -118,6 +145,9 @@ class LinearHead(Part):
         self.vocab, self.hidden = int(spec["vocab_size"]), int(spec["hidden_size"])
         self.name = spec["name"]
         self.tied_to = spec.get("tied_to")
+        self.softcap = float(spec["softcap"]) if spec.get("softcap") is not None else None
+        if self.softcap is not None and self.softcap <= 0:
+            raise ValueError(f"a softcap is positive, got {self.softcap}")
         self.linear = Linear(runtime, self.hidden, [self.vocab], [self.name])
 
     def tensors(self, prefix=""):
@@ -136,11 +166,15 @@ class LinearHead(Part):
 
     def forward(self, x: torch.Tensor, logits: torch.Tensor) -> torch.Tensor:
         """x [rows, hidden] -> logits float32 [rows, vocab]."""
-        return self.linear.forward(x, logits)
+        self.linear.forward(x, logits)
+        if self.softcap is not None:
+            self.rt.kernels.softcap(logits, self.softcap)
+        return logits
 
 
 register_part("embedding", "embedding", Embedding)
 register_part("embedding", "pair_hash_embedding", PairHashEmbedding)
 register_part("embedding", "normed_embedding", NormedEmbedding)
+register_part("embedding", "positioned_embedding", PositionedEmbedding)
 register_part("embedding", "row_table", RowTable)
 register_part("head", "linear_head", LinearHead)

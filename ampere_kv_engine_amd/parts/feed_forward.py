@@ -2,7 +2,8 @@
 down( silu(x Wg^T) * (x Wu^T) ), silu on the gate only.  Gate and up are one product: where the kernel set can, it
 also applies the activation before anything is stored (`gated_linear`); otherwise the stacked product is followed
 by the `swiglu` kernel.  With `activation="gelu_tanh"` the gate passes the tanh form of gelu instead of silu: the stacked
-product, then the activation kernel that takes either (`gated_activation`)."""
+product, then the activation kernel that takes either (`gated_activation`).  With `activation="clamped"` (`limit`, `slope`,
+`shift`): g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(slope * g) * (u + shift), by the same kernel."""
 
 from __future__ import annotations
 
@@ -22,8 +23,13 @@ class SwiGLU(Part):
         self.inter = int(spec["intermediate_size"])
         self.name = spec.get("name", "mlp")
         self.activation = spec.get("activation", "silu")
-        if self.activation not in ("silu", "gelu_tanh"):
-            raise ValueError(f"a gated feed-forward's activation is 'silu' or 'gelu_tanh', not {self.activation!r}")
+        if self.activation not in ("silu", "gelu_tanh", "clamped"):
+            raise ValueError(f"a gated feed-forward's activation is 'silu', 'gelu_tanh' or 'clamped', not {self.activation!r}")
+        self.constants = {}
+        if self.activation == "clamped":
+            self.constants = {name: float(spec[name]) for name in ("limit", "slope", "shift")}
+            if self.constants["limit"] <= 0:
+                raise ValueError(f"the limit of a clamped feed-forward is positive, got {self.constants['limit']}")
         gate, up, down = spec.get("names", ("gate_proj.weight", "up_proj.weight", "down_proj.weight"))
         self.gate_up = Linear(runtime, self.hidden, [self.inter, self.inter], [gate, up])
         self.down = Linear(runtime, self.inter, [self.hidden], [down])
@@ -67,7 +73,7 @@ class SwiGLU(Part):
             if self.activation == "silu":
                 self.rt.kernels.swiglu(gate_up, act)
             else:
-                self.rt.kernels.gated_activation(gate_up, act, self.activation)
+                self.rt.kernels.gated_activation(gate_up, act, self.activation, **self.constants)
         if ctx.fold_into_stream:     # the down product adds itself to the residual sum
             sums = self.down.add_to_stream(act, ctx)
             if sums is not None:

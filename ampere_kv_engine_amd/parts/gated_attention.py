@@ -14,6 +14,10 @@
     position (after the norm, where there is one; pairs in halves or interleaved, as the specification says), inside the
     kernel that writes the keys to their pages
     head h's output times sigmoid(w_g[h] . h), one number per head and token (`head_gate`), before W_o.
+    with `query_temperature` (coef, every): q times 1 + coef ln(floor((p + 1) / every) + 1) at position p
+    with `value_norm_eps`: every head's value divided by its root mean square (no weight) before it is cached
+    with `distance_bias`: score - r1_h ln(1 + r2_h (i - j)), after the softcap (tensors `r1`, `r2`, a number per head, kept
+    float32)
 
 Keys are `head_dim` wide, values `value_dim`; query head h reads kv head h // (q_heads / kv_heads).  Keys are cached
 after their norm.  All five projections are one product over the layer's input.
@@ -54,6 +58,14 @@ class GatedAttention(Part, SharesProducts):
         if self.keep_first < 0 or (self.keep_first and spec.get("window") is None):
             raise ValueError("kept first tokens come with a window, and their number is not negative")
         self.q_norm_weight = self.k_norm_weight = None
+        self.value_eps = float(spec["value_norm_eps"]) if spec.get("value_norm_eps") is not None else None
+        self.temperature = spec.get("query_temperature")
+        if self.temperature is not None:
+            self.temperature = (float(self.temperature[0]), int(self.temperature[1]))
+            if self.temperature[1] <= 0:
+                raise ValueError(f"a query temperature grows every so many positions, got {self.temperature[1]}")
+        self.has_bias = bool(spec.get("distance_bias", False))
+        self.distance_bias = None
         self.head_gate = bool(spec.get("head_gate", False))
         self.name = spec.get("name", "attn")
         if self.q_heads % self.kv_heads:
@@ -64,7 +76,7 @@ class GatedAttention(Part, SharesProducts):
         if self.softcap is not None and self.softcap <= 0:
             raise ValueError(f"softcap must be positive or None, got {self.softcap}")
         self.q_size, self.k_size, self.v_size = self.q_heads * self.dim, self.kv_heads * self.dim, self.kv_heads * self.vdim
-        names = dict(q="q", k="k", v="v", g="g", o="o", sink="sink")
+        names = dict(q="q", k="k", v="v", g="g", o="o", sink="sink", r1="r1", r2="r2")
         names.update(spec.get("names") or {})
         self.names = names
         bias = spec.get("bias_suffix")           # q, k and v have bias vectors named after them, with this suffix
@@ -77,7 +89,7 @@ class GatedAttention(Part, SharesProducts):
                 biases.append(None)
         self.width = sum(sizes)
         self.qkvg = self.inputs = Linear(runtime, self.hidden, sizes, stacked, bias_names=biases)
-        if self.learned_sink:
+        if self.learned_sink or self.has_bias:
             self.inputs = None      # (a tensor of its own beside the products: side by side with others it runs by itself)
         self.out = self.outputs = Linear(runtime, self.q_heads * self.vdim, [self.hidden], [names["o"]])
         runtime.kernels.check_gated_attention_sizes(self.q_heads, self.kv_heads, self.dim, self.vdim, runtime.page_size)
@@ -88,6 +100,9 @@ class GatedAttention(Part, SharesProducts):
     def _sink_spec(self, p):
         return [TensorSpec(p + self.names["sink"], (self.q_heads,), BIAS)] if self.learned_sink else []
 
+    def _bias_specs(self, p):
+        return [TensorSpec(p + self.names[n], (self.q_heads,), BIAS) for n in ("r1", "r2")] if self.has_bias else []
+
     def _norm_specs(self, p):
         if self.projection_eps is None:
             return []
@@ -96,7 +111,7 @@ class GatedAttention(Part, SharesProducts):
 
     def tensors(self, prefix):
         p = self._prefix(prefix)
-        return self.qkvg.tensors(p) + self.out.tensors(p) + self._sink_spec(p) + self._norm_specs(p)
+        return self.qkvg.tensors(p) + self.out.tensors(p) + self._sink_spec(p) + self._norm_specs(p) + self._bias_specs(p)
 
     def load(self, fetch, prefix):
         p = self._prefix(prefix)
@@ -104,6 +119,8 @@ class GatedAttention(Part, SharesProducts):
         self.out.load(fetch, p)
         if self.learned_sink:
             self.sink_logits = fetch(self._sink_spec(p)[0]).to(torch.float32).contiguous()
+        if self.has_bias:
+            self.distance_bias = torch.stack([fetch(spec).to(torch.float32) for spec in self._bias_specs(p)]).contiguous()
         if self.projection_eps is not None:
             self.q_norm_weight, self.k_norm_weight = (fetch(spec).to(torch.float32).contiguous()
                                                       for spec in self._norm_specs(p))
@@ -129,11 +146,17 @@ class GatedAttention(Part, SharesProducts):
         if self.projection_eps is not None:
             eps = self.projection_eps
             rotation.update(q_weight=self.q_norm_weight, k_weight=self.k_norm_weight, whole=True)
+        if self.value_eps is not None:
+            rotation["value_eps"] = self.value_eps
+        if self.temperature is not None:
+            rotation.update(temperature=self.temperature, positions=ctx.positions)
         k.unit_norm_write(projected, self.q_heads, self.kv_heads, self.dim, self.vdim, eps,
                           meta.slot_map if writes_cache else None, cache.k, cache.v, q, at=at, **rotation)
         more = {"sink_logits": self.sink_logits} if self.learned_sink else {}
         if self.keep_first:
             more["keep_first"] = self.keep_first
+        if self.has_bias:
+            more["distance_bias"] = self.distance_bias
         k.gated_attention(q, cache.k, cache.v, projected if self.head_gate else None,
                           at + self.q_size + self.k_size + self.v_size, ctx, meta, self.q_heads, self.kv_heads, self.dim,
                           self.vdim, self.scale, self.softcap, self.chunk, self.window, self.sink, out, out_at=out_at,

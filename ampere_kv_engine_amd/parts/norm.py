@@ -9,7 +9,10 @@ with the norm that follows (`after`): the norm kernel of blocks that norm a bran
 
 With `unit_offset` the file stores the weight around zero and the norm multiplies by 1 + w; the sum is formed once, at
 load, in float32.  With `output_scale` the normed rows are multiplied by a constant as well (a model whose logits are
-its head's product times a constant puts it on its final norm): the weight takes it once, at load, in float32."""
+its head's product times a constant puts it on its final norm): the weight takes it once, at load, in float32.
+
+With `scalar` the norm has ONE weight for all coordinates, stored as a tensor without axes; the vector the kernels read is
+filled with it once, at load."""
 
 from __future__ import annotations
 
@@ -17,7 +20,7 @@ import torch
 
 from ..weights.random import NORM_STD, _normal, register_init_law
 from ..weights.spec import NORM, TensorSpec
-from .base import Norm, NormedDelta, ScaledDelta, StreamSums, UnnormedRows, register_part  # noqa: F401  (StreamSums is found here too)
+from .base import Norm, NormedDelta, NormedPair, ScaledDelta, StreamSums, UnnormedRows, register_part  # noqa: F401  (StreamSums is found here too)
 
 
 NORM_OFFSET = "norm_offset"          # a norm weight that is stored around zero and applied as 1 + w
@@ -31,6 +34,7 @@ class RMSNorm(Norm):
         self.single_rounding = bool(spec.get("single_rounding", False))
         self.unit_offset = bool(spec.get("unit_offset", False))
         self.output_scale = float(spec.get("output_scale", 1.0))
+        self.scalar = bool(spec.get("scalar", False))
         self.rt = runtime
         self.weight: torch.Tensor | None = None
 
@@ -39,10 +43,11 @@ class RMSNorm(Norm):
         return NORM_OFFSET if self.unit_offset else NORM
 
     def tensors(self, name: str):
-        return [TensorSpec(name, (self.size,), self.role)]
+        return [TensorSpec(name, () if self.scalar else (self.size,), self.role)]
 
     def load(self, fetch, name: str):
-        self.weight = fetch(TensorSpec(name, (self.size,), self.role)).to(torch.float32).contiguous()
+        self.weight = fetch(self.tensors(name)[0]).to(torch.float32)
+        self.weight = self.weight.expand(self.size).contiguous() if self.scalar else self.weight.contiguous()
         if self.unit_offset:
             self.weight += 1.0
         if self.output_scale != 1.0:
@@ -76,6 +81,10 @@ class RMSNorm(Norm):
         self.rt.kernels.norm_add_norm(stream, delta, self.weight, self.eps, None, 0.0, None)
 
     def after(self, stream, pending, out):
+        if isinstance(pending, NormedPair) and self.single_rounding:       # one kernel: norm both branches, add, norm
+            self.rt.kernels.norm_add_norm(stream, pending.delta, pending.weight, pending.eps, self.weight, self.eps, out,
+                                          delta_scale=pending.scale, delta2=pending.second, post_weight2=pending.second_weight)
+            return out
         if isinstance(pending, ScaledDelta) and self.single_rounding:      # one kernel: add the branch times its constant, norm
             more = {"delta2": pending.second} if pending.second is not None else {}
             self.rt.kernels.norm_add_norm(stream, pending.delta, None, 0.0, self.weight, self.eps, out,

@@ -268,8 +268,11 @@ class TorchKernels(KernelSet):
         words[ctx.seq_slots.long(), 7] = cur[ctx.q_start.long()[1:] - 1].int()
 
     def norm_add_norm(self, stream, delta, post_weight, post_eps, pre_weight, pre_eps, out, delta_scale=1.0, offset=None,
-                      delta2=None):
-        if delta is not None:
+                      delta2=None, post_weight2=None):
+        if post_weight2 is not None:       # two branches, each normed by itself
+            unit = lambda v: v * torch.rsqrt((v * v).mean(-1, keepdim=True) + post_eps)
+            stream += delta_scale * (unit(delta.float()) * post_weight + unit(delta2.float()) * post_weight2)
+        elif delta is not None:
             d = (delta.float() + delta2.float() if delta2 is not None else delta.float()) * delta_scale
             if post_weight is not None:
                 d = d * torch.rsqrt((d * d).mean(-1, keepdim=True) + post_eps) * post_weight
@@ -284,6 +287,16 @@ class TorchKernels(KernelSet):
         rows = torch.empty_like(out)
         self.embed(ids, table, rows, ctx)
         out += rows
+
+    def embed_scaled(self, ids, table, scale, places, out, ctx):
+        """out[n] = table[id] * scale (+ places[position])."""
+        self.embed(ids, table, out, ctx)
+        out.mul_(scale)
+        if places is not None:
+            out += places[ctx.positions.long()].float()
+
+    def softcap(self, values, cap):
+        values.copy_(cap * torch.tanh(values / cap))
 
     def norm_gate_rows(self, x, weight, eps, gates, gate_at, gate, out, out_at=0, out_scale=1.0, x_at=0, width=None):
         width = x.shape[1] - x_at if width is None else width
@@ -302,9 +315,13 @@ class TorchKernels(KernelSet):
         self.embed(ids, table, out, ctx)
         out.copy_(out * torch.rsqrt((out * out).mean(-1, keepdim=True) + eps) * weight)
 
-    def gated_activation(self, gate_up, out, activation):
+    def gated_activation(self, gate_up, out, activation, limit=0.0, slope=1.0, shift=0.0):
         inter = out.shape[1]
         gate, up = gate_up[:, :inter].float(), gate_up[:, inter:].float()
+        if activation == "clamped":
+            gate, up = gate.clamp(max=limit), up.clamp(-limit, limit) + shift
+            out.copy_((gate * torch.sigmoid(slope * gate) * up).to(out.dtype))
+            return
         if activation == "gelu_tanh":
             act = 0.5 * gate * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (gate + 0.044715 * gate ** 3)))
         else:
@@ -323,8 +340,9 @@ class TorchKernels(KernelSet):
         assert heads % groups == 0
 
     def delta_rule(self, conv, beta_logits, beta_at, decay_logits, decay_bias, rate, gates, norm_weight, unit_eps, norm_eps,
-                   q_scale, heads, groups, dim, vdim, state, ctx, out):
-        """S of a request lies at the start of its slot as [heads, vdim, dim]."""
+                   q_scale, heads, groups, dim, vdim, state, ctx, out, decay_at=None, gate_at=0, gate="sigmoid"):
+        """S of a request lies at the start of its slot as [heads, vdim, dim].  `decay_at`: one decay a head, from columns
+        of `decay_logits`, and gates from columns of `gates`."""
         n = conv.shape[0]
         x = conv.float()
         qk = groups * dim
@@ -335,8 +353,13 @@ class TorchKernels(KernelSet):
         share = heads // groups
         q, k = q.repeat_interleave(share, dim=1), k.repeat_interleave(share, dim=1)
         beta = torch.sigmoid(beta_logits[:, beta_at:beta_at + heads].float())
-        g = torch.exp(-rate[None, :, None] * torch.nn.functional.softplus(
-            (decay_logits + decay_bias).view(n, heads, dim), threshold=20.0))
+        if decay_at is not None:
+            logits = (decay_logits[:, decay_at:decay_at + heads].float() + decay_bias)[:, :, None].expand(n, heads, dim)
+            gates = gates[:, gate_at:gate_at + heads * vdim].float()
+        else:
+            logits = (decay_logits + decay_bias).view(n, heads, dim)
+        g = torch.exp(-rate[None, :, None] * torch.nn.functional.softplus(logits, threshold=20.0))
+        opened = torch.sigmoid(gates) * (gates if gate == "silu" else 1.0)
         for r in range(ctx.num_seqs):
             first, last, slot = ctx.host_q_start[r], ctx.host_q_start[r + 1], ctx.host_seq_slots[r]
             S = state[slot, :heads * dim * vdim].view(heads, vdim, dim).transpose(1, 2).clone()      # [heads, dim, vdim]
@@ -346,8 +369,65 @@ class TorchKernels(KernelSet):
                 S = S + k[t][:, :, None] * u[:, None, :]
                 o = torch.einsum("hdv,hd->hv", S, q[t])
                 o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + norm_eps) * norm_weight
-                out[t] = (o * torch.sigmoid(gates[t].view(heads, vdim))).reshape(-1).to(out.dtype)
+                out[t] = (o * opened[t].view(heads, vdim)).reshape(-1).to(out.dtype)
             state[slot, :heads * dim * vdim] = S.transpose(1, 2).reshape(-1)
+
+    # ---- time mixing and the matrix memory ---------------------------------------------------------------------------
+    def check_state_sizes(self, heads, dim, vdim):
+        pass
+
+    def token_shift(self, x, mu, state, kept_at, ctx, out):
+        """out[s, t] = x_t + (x_(t-1) - x_t) * mu[s]; the row before a portion lies in the request's slot."""
+        for r in range(ctx.num_seqs):
+            first, last, slot = ctx.host_q_start[r], ctx.host_q_start[r + 1], ctx.host_seq_slots[r]
+            rows = x[first:last].float()
+            before = torch.cat((state[slot, kept_at:kept_at + x.shape[1]][None], rows[:-1]))
+            out[:, first:last] = (rows + (before - rows) * mu[:, None, :]).to(out.dtype)
+
+    def tanh_rows(self, x, out):
+        out.copy_(torch.tanh(x).to(out.dtype))
+
+    def time_mixing(self, rkvg, decay_logits, decay_bias, bonus, norm_weight, eps, x, heads, dim, state, kept_at, ctx, out):
+        """S of a request lies at the start of its slot as [heads, value, key], the last row of x from kept_at on."""
+        n = x.shape[0]
+        r_, k_, v_ = (rkvg[i].float().view(n, heads, dim) for i in range(3))
+        keep = torch.exp(-torch.exp(decay_logits + decay_bias)).view(n, heads, dim)
+        gate = rkvg[3].float()
+        for r in range(ctx.num_seqs):
+            first, last, slot = ctx.host_q_start[r], ctx.host_q_start[r + 1], ctx.host_seq_slots[r]
+            S = state[slot, :heads * dim * dim].view(heads, dim, dim).transpose(1, 2).clone()        # [heads, key, value]
+            for t in range(first, last):
+                o = torch.einsum("hdv,hd->hv", S, r_[t]) + (r_[t] * bonus.view(heads, dim) * k_[t]).sum(-1, keepdim=True) * v_[t]
+                S = keep[t][:, :, None] * S + k_[t][:, :, None] * v_[t][:, None, :]
+                o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)
+                out[t] = (o.reshape(-1) * norm_weight * gate[t] * torch.sigmoid(gate[t])).to(out.dtype)
+            state[slot, :heads * dim * dim] = S.transpose(1, 2).reshape(-1)
+            state[slot, kept_at:kept_at + x.shape[1]] = x[last - 1].float()
+
+    def matrix_memory(self, projected, i_bias, f_bias, cap, read_eps, norm_weight, eps, heads, dim, vdim, state, top_at, ctx, out):
+        """In the slot: [heads, vdim + 1, dim], a head's last row being n; the heads' running maxima from top_at on."""
+        n = projected.shape[0]
+        q, k, v, g, i, f = projected.float().split([heads * dim, heads * dim, heads * vdim, heads * vdim, heads, heads], dim=1)
+        q, k, v = q.reshape(n, heads, dim) * dim ** -0.5, k.reshape(n, heads, dim), v.reshape(n, heads, vdim)
+        v = torch.cat((v, torch.ones(n, heads, 1)), dim=-1)
+        into = cap * torch.tanh((i + i_bias) / cap)
+        keep = torch.nn.functional.logsigmoid(cap * torch.tanh((f + f_bias) / cap))
+        size = heads * dim * (vdim + 1)
+        for r in range(ctx.num_seqs):
+            first, last, slot = ctx.host_q_start[r], ctx.host_q_start[r + 1], ctx.host_seq_slots[r]
+            S = state[slot, :size].view(heads, vdim + 1, dim).transpose(1, 2).clone()
+            top = state[slot, top_at:top_at + heads].clone()
+            for t in range(first, last):
+                new = torch.maximum(keep[t] + top, into[t])
+                S = torch.exp(keep[t] + top - new)[:, None, None] * S + (torch.exp(into[t] - new)[:, None, None]
+                                                                         * k[t][:, :, None] * v[t][:, None, :])
+                top = new
+                o = torch.einsum("hdv,hd->hv", S, q[t])
+                o = o[:, :vdim] / (torch.maximum(o[:, vdim:].abs(), torch.exp(-top)[:, None]) + read_eps)
+                o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)
+                out[t] = (o.reshape(-1) * norm_weight * torch.sigmoid(g[t])).to(out.dtype)
+            state[slot, :size] = S.transpose(1, 2).reshape(-1)
+            state[slot, top_at:top_at + heads] = top
 
     @staticmethod
     def _turn(x, positions, table, rot_dims, interleaved=False):
@@ -455,7 +535,8 @@ class TorchKernels(KernelSet):
         pass
 
     def unit_norm_write(self, projected, q_heads, kv_heads, dim, vdim, eps, slot_map, k_pages, v_pages, q_out, at=0, maps=1,
-                        table=None, rot_dims=0, positions=None, q_weight=None, k_weight=None, whole=False, interleaved=False):
+                        table=None, rot_dims=0, positions=None, q_weight=None, k_weight=None, whole=False, interleaved=False,
+                        value_eps=None, temperature=None):
         projected = projected[:, at:]
         n = projected.shape[0]
         q_size, k_size, v_size = q_heads * maps * dim, kv_heads * maps * dim, kv_heads * vdim
@@ -470,6 +551,11 @@ class TorchKernels(KernelSet):
             q = q * q_weight.view(q_heads * maps, dim)
         if k_weight is not None:
             k = k * k_weight.view(kv_heads * maps, dim)
+        if temperature is not None:
+            coef, every = temperature
+            q = q * (1.0 + coef * torch.log(((positions.long() + 1) // every + 1).float()))[:, None, None]
+        if value_eps is not None:
+            v = v.float() * torch.rsqrt((v.float() ** 2).mean(-1, keepdim=True) + value_eps)
         if table is not None:
             q, k = self._turn(q, positions, table, rot_dims, interleaved), self._turn(k, positions, table, rot_dims, interleaved)
         q_out.copy_(q.reshape(n, q_size).to(q_out.dtype))
@@ -480,7 +566,8 @@ class TorchKernels(KernelSet):
             v_pages[slots // page_size, :, :, slots % page_size] = v.to(v_pages.dtype)
 
     def gated_attention(self, q, k_pages, v_pages, gates, gate_at, ctx, meta, q_heads, kv_heads, dim, vdim, scale, softcap,
-                        chunk, window, sink, out, out_at=0, out_scale=1.0, sink_logits=None, maps=1, keep_first=0):
+                        chunk, window, sink, out, out_at=0, out_scale=1.0, sink_logits=None, maps=1, keep_first=0,
+                        distance_bias=None):
         """`maps` > 1: a head has `maps` query vectors; vector number m of a head reads the m-th `dim` columns of its key
         head's record and the head's values.  `sink_logits`: the sink's term is exp(sink_logits[head])."""
         page_size = k_pages.shape[2]
@@ -518,6 +605,9 @@ class TorchKernels(KernelSet):
                 scores = (qs[:, head] @ record[:, head % maps * dim:head % maps * dim + dim].T) * scale
                 if softcap is not None:
                     scores = softcap * torch.tanh(scores / softcap)
+                if distance_bias is not None:
+                    apart = (q_pos[:, None] - key_pos[None, :]).clamp(min=0).float()
+                    scores = scores - distance_bias[0, head] * torch.log1p(distance_bias[1, head] * apart)
                 scores = scores.masked_fill(~visible, -math.inf)
                 top = scores.amax(-1, keepdim=True)
                 sunk = float(sink_logits[head]) if sink_logits is not None else 0.0
