@@ -27,9 +27,13 @@ from __future__ import annotations
 
 import torch
 
+from ..weights.random import register_init_law
 from ..weights.spec import BIAS, NORM, TensorSpec
 from .base import PagedKV, Part, SharesProducts, build_part, register_part
 from .linear import Linear
+
+DISTANCE_BIAS = "distance_bias"      # a distance bias's size and rate: never negative (the logarithm's argument stays above 1)
+register_init_law(DISTANCE_BIAS, lambda shape, generator, device: torch.rand(shape, generator=generator, dtype=torch.float32, device=device))
 
 
 class GatedAttention(Part, SharesProducts):
@@ -101,7 +105,7 @@ class GatedAttention(Part, SharesProducts):
         return [TensorSpec(p + self.names["sink"], (self.q_heads,), BIAS)] if self.learned_sink else []
 
     def _bias_specs(self, p):
-        return [TensorSpec(p + self.names[n], (self.q_heads,), BIAS) for n in ("r1", "r2")] if self.has_bias else []
+        return [TensorSpec(p + self.names[n], (self.q_heads,), DISTANCE_BIAS) for n in ("r1", "r2")] if self.has_bias else []
 
     def _norm_specs(self, p):
         if self.projection_eps is None:

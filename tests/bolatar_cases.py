@@ -52,12 +52,16 @@ BOLATAR_C = dict(
         dict(type="delta", mixer=DELTA(4, 2, 64, 128, 4), mlp=DENSE(128, 1.2)),
         dict(type="parallel", mixer=PARALLEL(LEFT(2, 1, 128, 64, 0.1, 0.25, 64), RIGHT(4, 32, 8)), mlp=None),
     ])
-BOLATAR = {"A": (BOLATAR_A, 81, 4), "B": (BOLATAR_B, 82, 8), "C": (BOLATAR_C, 83, 16)}        # config, weight seed, page size
+BOLATAR = {"A": (BOLATAR_A, 81, 4), "B": (BOLATAR_B, 84, 8), "C": (BOLATAR_C, 83, 16)}        # config, weight seed, page size
 
 LENGTHS, PROMPTS, POOL_TOKENS = K.LENGTHS, K.PROMPTS, K.POOL_TOKENS
-# float32: a few hundred float32 operations and recurrences over two hundred tokens.  bfloat16: as served, against the plain
-# float32 logits.
-LIMITS = {"float32": dict(max=2e-4, rms=2e-4), "bfloat16": dict(max=0.08, rms=0.1)}
+# float32: a few hundred float32 operations and recurrences over two hundred tokens; measured up to 4e-6 (1e-4 in a
+# drawn configuration whose softmaxes are very sharp).  bfloat16: as served,
+# against the plain float32 logits: positions lie within 0.04 (median 0.003 to 0.008) - except where a head's read-out is
+# almost zero before it is normed (a first token whose query and key are nearly at right angles: its sign and size are then
+# rounding; the torch double, which rounds where the kernels round, shows the same): a twentieth of a request's positions may
+# lie beyond.
+LIMITS = {"float32": dict(max=3e-4, rms=3e-4), "bfloat16": dict(max=0.06, rms=0.08)}
 BEYOND = {"float32": 0.0, "bfloat16": 0.05}
 
 
@@ -160,6 +164,14 @@ def check(engine, case, schedule):
     assert engine.cache.slots.num_free == engine.config.max_seqs, "slots were lost"
     print(f"[bolatar {case['name']} {dtype}] worst error {worst:.2f} of its limit")
     return pages
+
+
+def spread(got: dict, case) -> tuple[float, float]:
+    """(median, 90th percentile) over all requests' positions of the worst logit's error against the largest |logit|."""
+    errors = [(got[name] - want).abs().amax(1) / want.abs().max() for name, want in case["expected"].items()]
+    errors = torch.cat(errors)
+    assert not torch.isnan(errors).any(), "NaN logits"
+    return float(errors.median()), float(errors.quantile(0.9))
 
 
 # ---- the cuttings (those of the other designs' cases, held to this design's limits) -----------------------------------

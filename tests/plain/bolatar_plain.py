@@ -119,6 +119,19 @@ def shifted(h: torch.Tensor) -> torch.Tensor:
     return torch.cat((torch.zeros_like(h[:1]), h[:-1]))
 
 
+def mixed_states(r, k, v, keep, bonus) -> torch.Tensor:
+    """r, k, v, keep [n, heads, dim], bonus [heads, dim] -> the read-outs before their norm."""
+    n, heads, dim = r.shape
+    out = torch.empty(n, heads, dim, dtype=r.dtype)
+    for head in range(heads):
+        state = torch.zeros(dim, dim, dtype=r.dtype)
+        for t in range(n):
+            write = torch.outer(k[t, head], v[t, head])
+            out[t, head] = (state + bonus[head][:, None] * write).T @ r[t, head]
+            state = keep[t, head][:, None] * state + write
+    return out
+
+
 def time_mixing(h: torch.Tensor, w: dict, m: dict, eps: float) -> torch.Tensor:
     n = h.shape[0]
     heads, dim = m["heads"], m["dim"]
@@ -126,13 +139,7 @@ def time_mixing(h: torch.Tensor, w: dict, m: dict, eps: float) -> torch.Tensor:
     r, k, v = ((mixed[s] @ w[s].T).view(n, heads, dim) for s in "rkv")
     gate = silu(mixed["g"] @ w["g"].T)
     keep = torch.exp(-torch.exp(torch.tanh(mixed["w"] @ w["w1"].T) @ w["w2"].T + w["w0"])).view(n, heads, dim)
-    out = torch.empty(n, heads, dim, dtype=h.dtype)
-    for head in range(heads):
-        state = torch.zeros(dim, dim, dtype=h.dtype)
-        for t in range(n):
-            write = torch.outer(k[t, head], v[t, head])
-            out[t, head] = (state + w["u"][head][:, None] * write).T @ r[t, head]
-            state = keep[t, head][:, None] * state + write
+    out = mixed_states(r, k, v, keep, w["u"])
     return (unit_rms(out, eps).reshape(n, heads * dim) * w["norm"] * gate) @ w["o"].T
 
 

@@ -162,15 +162,25 @@ def random_configuration(seed: int) -> tuple:
 @pytest.mark.filterwarnings("ignore:a bfloat16 matrix")
 @pytest.mark.parametrize("seed", range(800, 810))
 def test_a_random_configuration_through_the_cuttings(seed, tmp_path):
+    """float32 against the plain implementation, position by position.  In bfloat16 a drawn configuration may amplify rounding
+    (softmaxes of a few keys, read-outs near zero that are normed): its errors are held to those of the torch double, which
+    rounds where the kernels round."""
+    from torch_kernels import TorchKernels
     config = random_configuration(seed)
     print(f"seed {seed}: {config[0]}, pages of {config[2]}", flush=True)
     case = B.make_case(f"random {seed}", str(tmp_path), config)
-    for dtype in ("float32", "bfloat16"):
-        engine = B.make_engine(case, dtype, DEVICE)
-        B.case_whole(engine, case)
-        B.case_portions_down_to_two_tokens(engine, case)
-        B.case_prefill_then_token_by_token(engine, case)
-        B.case_mixed_with_pages_and_slots_used_again(engine, case)
+    engine = B.make_engine(case, "float32", DEVICE)
+    B.case_whole(engine, case)
+    B.case_portions_down_to_two_tokens(engine, case)
+    B.case_prefill_then_token_by_token(engine, case)
+    B.case_mixed_with_pages_and_slots_used_again(engine, case)
+    double = B.make_engine(case, "bfloat16", "cpu", kernels=TorchKernels())
+    allowed = B.spread(schedules.run(double, case["requests"], schedules.whole(case["requests"]))[0], case)
+    engine = B.make_engine(case, "bfloat16", DEVICE)
+    for schedule in (schedules.whole(case["requests"]), schedules.portions(case["requests"]), schedules.last_one_by_one(case["requests"], 32),
+                     schedules.mixed(case["requests"], B.PROMPTS, case["page_size"], engine.config.num_pages, seed=5, max_live=3)):
+        got = B.spread(schedules.run(engine, case["requests"], schedule)[0], case)
+        assert all(g <= 1.5 * a + 0.004 for g, a in zip(got, allowed)), f"bfloat16 (median, 90 %) {got}, the double {allowed}"
 
 
 LONG = {
@@ -346,6 +356,7 @@ def test_time_mixing_alone(hip, dtype, heads, dim, width, rank):
     kept_at = heads * dim * dim
     state = torch.zeros(4, kept_at + width, device=DEVICE)
     mu = torch.stack([w[f"mu.{s}"] for s in "rkvgw"]).to(DEVICE)
+    inputs = []               # what the recurrence was given, step by step: in bfloat16 it is held to its rounded inputs
 
     def run(ctx, cut):
         x = cut([r.to(dtype) for r in rows])
@@ -357,7 +368,9 @@ def test_time_mixing_alone(hip, dtype, heads, dim, width, rank):
         low = torch.empty(n, rank, dtype=torch.float32, device=DEVICE)
         hip.tanh_rows(down, low)
         out = torch.empty(n, wide, dtype=dtype, device=DEVICE)
-        hip.time_mixing(rkvg, low @ w["w2"].T.to(DEVICE), w["w0"].to(DEVICE), w["u"].reshape(-1).to(DEVICE), w["norm"].to(DEVICE), eps, x, heads,
+        logits = low @ w["w2"].T.to(DEVICE)
+        inputs.append((ctx.host_q_start, rkvg.float().cpu(), logits.cpu()))
+        hip.time_mixing(rkvg, logits, w["w0"].to(DEVICE), w["u"].reshape(-1).to(DEVICE), w["norm"].to(DEVICE), eps, x, heads,
                         dim, state, kept_at, ctx, out)
         return out
 
@@ -365,7 +378,13 @@ def test_time_mixing_alone(hip, dtype, heads, dim, width, rank):
     assert not state[0].any() and not state[2].any()
     for r, slot in enumerate((3, 1)):
         torch.testing.assert_close(state[slot, kept_at:].cpu(), rows[r][-1], rtol=0, atol=0)
-        _close(got[r], plain.time_mixing(rows[r], w, dict(heads=heads, dim=dim), eps), dtype, f32=1e-4, bf16=0.05)
+        if dtype == torch.float32:
+            _close(got[r], plain.time_mixing(rows[r], w, dict(heads=heads, dim=dim), eps), dtype, f32=1e-4)
+        given = torch.cat([x[:, q[r]:q[r + 1]] for q, x, _ in inputs], dim=1)
+        logits = torch.cat([x[q[r]:q[r + 1]] for q, _, x in inputs])
+        keep = torch.exp(-torch.exp(logits + w["w0"]))
+        raw = plain.mixed_states(*(x.reshape(-1, heads, dim) for x in (*given[:3], keep)), w["u"])
+        _close(got[r], plain.unit_rms(raw, eps).reshape(-1, wide) * w["norm"] * plain.silu(given[3]), dtype)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
