@@ -1,4 +1,4 @@
-"""Prefill and decode throughput of the Keranex design (and, `--workload tukevik` / `lirulix` / `mekuvik`, of those designs) at sizes that resemble a real model's layers (random weights),
+"""Prefill and decode throughput of the Keranex design (and, `--workload tukevik` / `lirulix` / `mekuvik` / `bolatar`, of those designs) at sizes that resemble a real model's layers (random weights),
 beside the dense Qwen3 decoder at equal width, depth, heads and active feed-forward width - the closest model the
 engine has.  `python bench.py --workload keranex [--design-sizes s,m] [--layers L]` prints one JSON line per size:
 
@@ -146,6 +146,30 @@ def mekuvik_config(size: dict, layers: int) -> dict:
                 loop=dict(start=0, stop=layers, times=1))
 
 
+# Bolatar at the same widths: the pattern [delta rule, attention beside time mixing, matrix memory, attention beside time
+# mixing], every layer with a dense feed-forward.  Beside it Lirulix at its size of the same name (the closest design the
+# engine has: the delta rule on the same walk, attention on the same kernels, dense feed-forwards of the same width) and Qwen3.
+BOLATAR_SIZES = {
+    "s": dict(width=2048, vocab=32768, d_heads=16, d_kv_heads=16, d_dim=128, d_vdim=128, conv=4, heads=16, kv_heads=4, dim=128, vdim=128,
+              t_heads=32, t_dim=64, rank=64, m_heads=16, m_dim=128, m_vdim=128, ff=3072),
+    "m": dict(width=4096, vocab=65536, d_heads=32, d_kv_heads=32, d_dim=128, d_vdim=128, conv=4, heads=32, kv_heads=8, dim=128, vdim=128,
+              t_heads=64, t_dim=64, rank=128, m_heads=32, m_dim=128, m_vdim=128, ff=5120),
+}
+
+
+def bolatar_config(size: dict, layers: int) -> dict:
+    delta = dict(heads=size["d_heads"], kv_heads=size["d_kv_heads"], dim=size["d_dim"], vdim=size["d_vdim"], conv=size["conv"])
+    both = dict(left=dict(heads=size["heads"], kv_heads=size["kv_heads"], dim=size["dim"], vdim=size["vdim"], scale=size["dim"] ** -0.5,
+                          q_temp=dict(coef=0.1, every=4096)),
+                right=dict(heads=size["t_heads"], dim=size["t_dim"], rank=size["rank"]))
+    memory = dict(heads=size["m_heads"], dim=size["m_dim"], vdim=size["m_vdim"], gate_cap=15.0)
+    mlp = dict(kind="dense", ff=size["ff"], limit=7.0)
+    pattern = [("delta", delta), ("parallel", both), ("mlstm", memory), ("parallel", both)]
+    return dict(architecture="Bolatar", vocab=size["vocab"], width=size["width"], max_positions=8192, norm=dict(eps=1e-6),
+                embedding=dict(scale=size["width"] ** 0.5), logit_softcap=30.0,
+                layers=[dict(type=kind, mixer=mixer, mlp=mlp) for kind, mixer in (pattern[i % 4] for i in range(layers))])
+
+
 def qwen3_beside_tukevik(size: dict, layers: int) -> dict:
     return dict(architectures=["Qwen3ForCausalLM"], num_hidden_layers=layers, hidden_size=size["width"],
                 num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=size["dim"],
@@ -212,7 +236,22 @@ def measure(config, batch: int, context: int, steps: int, warmup: int, graphs: b
 
 def design_workload(sizes: str, layers: int | None, batch: int, context: int, steps: int, warmup: int,
                     graphs: bool = True, only: str = "", design: str = "keranex") -> int:
-    from .config import KeranexConfig, LirulixConfig, MekuvikConfig, Qwen3Config, TukevikConfig
+    from .config import BolatarConfig, KeranexConfig, LirulixConfig, MekuvikConfig, Qwen3Config, TukevikConfig
+    for name in [s for s in sizes.split(",") if s and design == "bolatar"]:
+        size, beside = BOLATAR_SIZES[name], LIRULIX_SIZES[name]
+        count = layers or 8
+        line = {"workload": "bolatar", "sizes": name, "layers": count, "batch": batch, "context": context,
+                "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
+                "shape": size}
+        if only in ("", "bolatar"):
+            line["bolatar"] = measure(BolatarConfig.from_dict(bolatar_config(size, count)), batch, context, steps, warmup, graphs)
+        if only in ("", "lirulix"):
+            line["lirulix_equal_size"] = measure(LirulixConfig.from_dict(lirulix_config(beside, count)), batch, context, steps, warmup, graphs)
+        if only in ("", "qwen3"):
+            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_beside_tukevik(dict(beside, dense=beside["ff"]), count)), batch, context, steps, warmup, graphs)
+        print(json.dumps(line), flush=True)
+    if design == "bolatar":
+        return 0
     for name in [s for s in sizes.split(",") if s and design == "mekuvik"]:
         size, beside = MEKUVIK_SIZES[name], TUKEVIK_SIZES[name]
         count = layers or 8

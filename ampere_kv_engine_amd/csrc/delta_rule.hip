@@ -5,7 +5,7 @@
 // exponentials, the state and its sums, the norm of the outputs.
 //
 // Three kernels.  `delta_prepare` is token-wise: the unit vectors, decays, betas and k . q of every token, float32, into a
-// workspace.  The walk over a request's tokens is `state_walk_kernel` (state_walk.h) with the rule kDelta.
+// workspace.  The walk over a request's tokens is state_walk.h's with the rule kDelta.
 // `state_finish_kernel` is token-wise again: o / rms(o) times a weight per value channel and a gate.
 
 #include "api_parts.h"
@@ -74,7 +74,7 @@ int delta_rule(const T* conv, long conv_stride, const T* beta_logits, long beta_
                const int* q_start, const int* seq_slots, float* workspace, T* out, int tokens, int seqs, int heads, int groups,
                int dim, int vdim, int longest, hipStream_t stream) {
   float* prepared = workspace;
-  float* raw = workspace + static_cast<long>(tokens) * prepared_width(heads, groups, dim, HEAD_DECAY);
+  float* raw = workspace + (static_cast<long>(tokens) + kRowsBehind) * prepared_width(heads, groups, dim, HEAD_DECAY);
   const int units = groups + (HEAD_DECAY ? 0 : (heads * dim + 255) / 256);
   const dim3 prepare_grid(static_cast<unsigned>(tokens), static_cast<unsigned>((units + 3) / 4));
   delta_prepare_kernel<T, TD, HEAD_DECAY><<<prepare_grid, 256, 0, stream>>>(conv, conv_stride, beta_logits, beta_stride,
@@ -95,7 +95,7 @@ int delta_rule(const T* conv, long conv_stride, const T* beta_logits, long beta_
 extern "C" {
 
 long akv_delta_rule_workspace(int tokens, int heads, int groups, int dim, int vdim, int decay_per_head) {
-  return static_cast<long>(tokens) * (prepared_width(heads, groups, dim, decay_per_head != 0) + static_cast<long>(heads) * vdim);
+  return (static_cast<long>(tokens) + kRowsBehind) * (prepared_width(heads, groups, dim, decay_per_head != 0) + static_cast<long>(heads) * vdim);
 }
 
 int akv_delta_rule(const void* conv, long conv_stride, int dtype, const void* beta_logits, long beta_stride,

@@ -185,7 +185,7 @@ int time_mixing(const T* r, const T* k, const T* v, const T* gates, long row_str
                 float* state, long state_stride, long kept_at, const int* q_start, const int* seq_slots, float* workspace, T* out,
                 int tokens, int seqs, int heads, int dim, int longest, hipStream_t stream) {
   float* prepared = workspace;
-  float* raw = workspace + static_cast<long>(tokens) * prepared_width(heads, heads, dim, false);
+  float* raw = workspace + (static_cast<long>(tokens) + kRowsBehind) * prepared_width(heads, heads, dim, false);
   time_mixing_prepare_kernel<T><<<dim3(tokens + seqs, (heads + 3) / 4), 256, 0, stream>>>(
       r, k, row_stride, decay_logits, decay_bias, bonus, prepared, tokens, heads, dim, x, width, state, state_stride, kept_at,
       q_start, seq_slots);
@@ -205,7 +205,7 @@ int matrix_memory(const T* q, const T* k, const T* v, const T* gates, const T* i
                   float* workspace, T* out, int tokens, int seqs, int heads, int dim, int vdim, int longest,
                   hipStream_t stream) {
   float* prepared = workspace;
-  float* raw = prepared + static_cast<long>(tokens) * prepared_width(heads, heads, dim, true);
+  float* raw = prepared + (static_cast<long>(tokens) + kRowsBehind) * prepared_width(heads, heads, dim, true);
   float* tops = raw + static_cast<long>(tokens) * heads * (vdim + 1);
   const int threads = min(1024, (longest + kWave - 1) / kWave * kWave);
   matrix_memory_gates_kernel<T><<<dim3(seqs, heads), threads, 0, stream>>>(i_logits, f_logits, row_stride, i_bias, f_bias, cap,
@@ -248,7 +248,7 @@ int akv_tanh_rows(const float* x, void* out, int dtype, long count, hipStream_t 
 }
 
 long akv_time_mixing_workspace(int tokens, int heads, int dim) {
-  return static_cast<long>(tokens) * (prepared_width(heads, heads, dim, false) + static_cast<long>(heads) * dim);
+  return (static_cast<long>(tokens) + kRowsBehind) * (prepared_width(heads, heads, dim, false) + static_cast<long>(heads) * dim);
 }
 
 int akv_time_mixing(const void* r, const void* k, const void* v, const void* gates, int dtype, long row_stride,
@@ -269,7 +269,7 @@ int akv_time_mixing(const void* r, const void* k, const void* v, const void* gat
 }
 
 long akv_matrix_memory_workspace(int tokens, int heads, int dim, int vdim) {
-  return static_cast<long>(tokens) * (prepared_width(heads, heads, dim, true) + static_cast<long>(heads) * (vdim + 2));
+  return (static_cast<long>(tokens) + kRowsBehind) * (prepared_width(heads, heads, dim, true) + static_cast<long>(heads) * (vdim + 2));
 }
 
 int akv_matrix_memory(const void* q, const void* k, const void* v, const void* gates, const void* i_logits, const void* f_logits,
