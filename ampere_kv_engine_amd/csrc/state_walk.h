@@ -491,16 +491,14 @@ __global__ __launch_bounds__(THREADS) void tile_walk_kernel(const float* __restr
     const bool whole = filled && count == kTile;      // (the same for the whole block)
 #pragma unroll
     for (int j = 0; j < kFours; ++j) {
-      if (!whole) {
-        const bool there = group + j * kRowStep < count;
+      const bool there = whole || (group + j * kRowStep < count && my_d < dim);
 #pragma unroll
-        for (int a = 0; a < kArrays; ++a) {
-          const float other = a == 2 ? 1.f : 0.f;
-          if (!(there && my_d < dim)) next[a][j] = make_float4(other, other, other, other);
-        }
+      for (int a = 0; a < kArrays; ++a) {
+        const float other = a == 2 ? 1.f : 0.f;
+        const float4 v = next[a][j];
+        *reinterpret_cast<float4*>(at + j * kRowStep * kArrays * kArray + a * kArray) =
+            make_float4(there ? v.x : other, there ? v.y : other, there ? v.z : other, there ? v.w : other);
       }
-#pragma unroll
-      for (int a = 0; a < kArrays; ++a) *reinterpret_cast<float4*>(at + j * kRowStep * kArrays * kArray + a * kArray) = next[a][j];
     }
 #pragma unroll
     for (int j = 0; j < kValueLoads; ++j) {
@@ -654,7 +652,7 @@ int launch_state_walk(const float* prepared, const T* values, long value_stride,
         prepared, values, value_stride, state, state_stride, q_start, seq_slots, raw, units, heads, groups, dim, vdim, ones);   \
   } while (0)
     if (R == 64) AKV_TILES(64, 1, 256);
-    else if (R == 32) AKV_TILES(32, (RULE == kDelta ? 1 : 2), 256);
+    else if (R == 32) AKV_TILES(32, 1, 256);
     else if (R == 16) AKV_TILES(16, 1, 128);
     else AKV_TILES(8, 1, 128);
 #undef AKV_TILES
