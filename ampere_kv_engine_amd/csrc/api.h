@@ -41,7 +41,7 @@ int akv_linear_tiled(const void* x, int x_dtype, const void* w, int w_dtype, voi
 int akv_linear_packed(const void* x, const void* wp, void* y, int y_dtype, int rows, int outs, int k, int n_tiles,
                       int k_tiles, int x_packed, const float* bias, hipStream_t stream);
 int akv_linear_packed_swiglu(const void* x, const void* wp, void* y, int y_dtype, int rows, int inter, int k,
-                             int n_tiles, int k_tiles, int x_packed, hipStream_t stream);
+                             int n_tiles, int k_tiles, int x_packed, const float* clamp, hipStream_t stream);
 int akv_linear_packed_normed(const float* stream_in, const void* delta, const float* norm_weight, float eps,
                              float* stream_out, const void* wp, void* y, int rows, int outs, int k, int n_tiles,
                              int k_tiles, int gated, const float* bias, hipStream_t stream);

@@ -47,7 +47,7 @@ struct DecodeArgs {
   float* sums_out;          // ADDS: [n_tiles][16]
   bf16_t* rows_out;         // ADDS: [rows, outs] or null: the new residual sum times `gain_out`, for a ROWSCALED reader
   const float* gain_out;    // ADDS: [outs], the weight of the norm that follows (with rows_out)
-  const float* bias;        // [outs] or null: added to the sums over k before anything else is done with them (never GATED)
+  const float* bias;        // [outs] or null: added to the sums over k before anything else is done with them; GATED: `clamp` of `gate_times`
   float eps;
   int sum_tiles, rows, outs, k, k_tiles, n_tiles, k_split, red_floats;
   float* pieces;            // [wave-row][2][RT][4][64]: the sums of a wave-row whose parts of k lie in two blocks
@@ -329,7 +329,7 @@ __global__ __launch_bounds__(768) void linear_decode_kernel(const DecodeArgs a) 
       if (g == 0) a.sums_out[tile * 16 + r] = squares;
     }
   } else if constexpr (GATED) {
-    store_tile<bf16_t>(a.y, silu_times(acc[0], acc[1]), r, (row_tile >> 1) * 16 + g * 4, a.rows, a.outs);
+    store_tile<bf16_t>(a.y, gate_times(acc[0], acc[1], a.bias), r, (row_tile >> 1) * 16 + g * 4, a.rows, a.outs);
   } else {
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt)
@@ -473,8 +473,8 @@ extern "C" int akv_linear_adds_rows(const void* x, const void* wp, float* stream
                      rows_out, gain, stream);
 }
 
-// y [rows, outs] = (x W^T) with every row scaled by rsqrt(its mean of squares + eps), plus `bias` (gated: silu of
-// the scaled gate times the scaled up): x [rows, k] bfloat16 are the rows akv_linear_adds_rows left - the residual
+// y [rows, outs] = (x W^T) with every row scaled by rsqrt(its mean of squares + eps), plus `bias` (gated: what
+// `gate_times` makes of the scaled gate and the scaled up, `bias` being its `clamp`): x [rows, k] bfloat16 are the rows akv_linear_adds_rows left - the residual
 // sum times the norm's weight -, `sums` [sum_tiles][16] the partial sums of squares of the residual rows it left
 // (sum_tiles = ceil(k / 16)).  Sizes, `pieces`, `arrivals`, `row_tiles`: as for akv_linear_scaled, without its limit
 // on the rows' bytes.
@@ -484,7 +484,7 @@ extern "C" int akv_linear_rowscaled(const void* x, const float* sums, int sum_ti
                                     hipStream_t stream) {
   if (rows <= 0 || outs <= 0) return 0;
   if (rows > 16 || (k & 7) != 0 || k_tiles * 32 < k || sum_tiles != (k + 15) / 16) return -2;
-  if (row_tiles < 0 || row_tiles > 2 || (gated && (row_tiles == 1 || bias != nullptr))) return -2;
+  if (row_tiles < 0 || row_tiles > 2 || (gated && row_tiles == 1)) return -2;
   if (gated ? ((outs & 15) != 0 || n_tiles * 8 != outs) : n_tiles * 16 < outs) return -2;
   DecodeArgs a{};
   a.x = static_cast<const bf16_t*>(x);
@@ -511,14 +511,15 @@ extern "C" int akv_linear_rowscaled(const void* x, const float* sums, int sum_ti
 // [sum_tiles][16] (what akv_linear_adds left: sum_tiles = ceil(k / 16)).  rows <= 16, k % 8 == 0, and the normed rows
 // (rows * k bfloat16) fit into a compute unit's LDS (160 KB) beside 832 bytes; -2 otherwise.  `pieces`, `arrivals`: as
 // for akv_linear_adds.  `row_tiles`: row tiles per wave of the plain product, 1 or 2; 0 leaves the choice to the sizes (a
-// gated product's waves always take a pair).  `bias` [outs] float32 or null (never with `gated`): y = norm(stream) W^T + bias.
+// gated product's waves always take a pair).  `bias` [outs] float32 or null: y = norm(stream) W^T + bias
+// (gated: `clamp` in its place).
 extern "C" int akv_linear_scaled(const float* stream_in, const float* sums, int sum_tiles, const float* gain, float eps,
                                  const void* wp, void* y, float* pieces, unsigned int* arrivals, int exchange_tiles,
                                  int rows, int outs, int k, int n_tiles, int k_tiles, int gated, int row_tiles,
                                  const float* bias, hipStream_t stream) {
   if (rows <= 0 || outs <= 0) return 0;
   if (rows > 16 || (k & 7) != 0 || k_tiles * 32 < k || sum_tiles != (k + 15) / 16) return -2;
-  if (row_tiles < 0 || row_tiles > 2 || (gated && (row_tiles == 1 || bias != nullptr))) return -2;
+  if (row_tiles < 0 || row_tiles > 2 || (gated && row_tiles == 1)) return -2;
   if (gated ? ((outs & 15) != 0 || n_tiles * 8 != outs) : n_tiles * 16 < outs) return -2;
   DecodeArgs a{};
   a.stream = stream_in;

@@ -298,7 +298,7 @@ __global__ __launch_bounds__(512) void linear_skinny_kernel(const bf16_t* __rest
 #pragma unroll
       for (int mt = 0; mt < MT; ++mt)
         if (row_tile + rt < n_tiles)
-          store_tile<TY>(y, silu_times(acc[rt][mt], acc[rt + 1][mt]), mt * 16 + r, ((row_tile + rt) >> 1) * 16 + g * 4,
+          store_tile<TY>(y, gate_times(acc[rt][mt], acc[rt + 1][mt], bias), mt * 16 + r, ((row_tile + rt) >> 1) * 16 + g * 4,
                          rows, outs);
   } else {
 #pragma unroll
@@ -338,7 +338,7 @@ int launch_skinny(const void* x, const void* wp, void* y, int rows, int outs, in
   }
   linear_skinny_kernel<MT, RT, TY, GATED, NORMED><<<blocks, waves * 64, lds, stream>>>(
       static_cast<const bf16_t*>(x), static_cast<const uintx4*>(wp), static_cast<TY*>(y), rows, outs, k, k_tiles,
-      n_tiles, k_split, x_packed, norm, GATED ? nullptr : bias);
+      n_tiles, k_split, x_packed, norm, bias);
   return AKV_LAUNCH_STATUS();
 }
 
@@ -541,7 +541,7 @@ __global__ __launch_bounds__(256, 2) void linear_wide_kernel(const bf16_t* __res
     for (int n = 0; n < 4; n += 2)
 #pragma unroll
       for (int m = 0; m < MW; ++m)
-        store_tile<TY>(y, silu_times(acc[n][m], acc[n + 1][m]), token0 + wave_m * (16 * MW) + m * 16 + r,
+        store_tile<TY>(y, gate_times(acc[n][m], acc[n + 1][m], bias), token0 + wave_m * (16 * MW) + m * 16 + r,
                        ((tile0 + n) >> 1) * 16 + g * 4, rows, outs);
   } else {
 #pragma unroll
@@ -566,11 +566,11 @@ int launch_wide(const void* x, const void* wp, void* y, int rows, int outs, int 
   if (tall)
     linear_wide_kernel<TY, 8, GATED><<<static_cast<unsigned>(blocks), 256, 0, stream>>>(
         static_cast<const bf16_t*>(x), static_cast<const uintx4*>(wp), static_cast<TY*>(y), rows, outs, k, k_tiles,
-        n_tiles, n_blocks, m_blocks, GATED ? nullptr : bias);
+        n_tiles, n_blocks, m_blocks, bias);
   else
     linear_wide_kernel<TY, 4, GATED><<<static_cast<unsigned>(blocks), 256, 0, stream>>>(
         static_cast<const bf16_t*>(x), static_cast<const uintx4*>(wp), static_cast<TY*>(y), rows, outs, k, k_tiles,
-        n_tiles, n_blocks, m_blocks, GATED ? nullptr : bias);
+        n_tiles, n_blocks, m_blocks, bias);
   return AKV_LAUNCH_STATUS();
 }
 
@@ -666,12 +666,14 @@ extern "C" int akv_linear_packed_static(const void* x, const void* wp, void* y, 
 }
 
 // The gated pair in one pass: wp holds 2 * inter / 16 row tiles, gate tile t at 2t and up tile t at 2t + 1;
-// y [rows, inter] = silu(x Wgate^T) * (x Wup^T).  inter must be a multiple of 16.
+// y [rows, inter] = silu(x Wgate^T) * (x Wup^T), or with `clamp` (three numbers on the device, else null) the clamped gate
+// of `gate_times`.  inter must be a multiple of 16.
 extern "C" int akv_linear_packed_swiglu(const void* x, const void* wp, void* y, int y_dtype, int rows, int inter,
-                                        int k, int n_tiles, int k_tiles, int x_packed, hipStream_t stream) {
+                                        int k, int n_tiles, int k_tiles, int x_packed, const float* clamp,
+                                        hipStream_t stream) {
   if (rows <= 0 || inter <= 0) return 0;
   if ((k & 7) != 0 || (inter & 15) != 0 || n_tiles * 8 != inter || k_tiles * 32 < k) return -2;
-  return linear_packed<true>(x, wp, y, y_dtype, rows, inter, k, n_tiles, k_tiles, x_packed, stream);
+  return linear_packed<true>(x, wp, y, y_dtype, rows, inter, k, n_tiles, k_tiles, x_packed, stream, clamp);
 }
 
 
@@ -679,7 +681,7 @@ extern "C" int akv_linear_packed_swiglu(const void* x, const void* wp, void* y, 
 // (bfloat16 activations), normed by every block of the product for itself; stream_out [rows, k] receives
 // stream_in + delta and must be another buffer than stream_in.  `gated`: akv_linear_packed_swiglu's packing and result.
 // At most 4 rows; k a multiple of 8; -2 where the rows do not fit the block's LDS beside its sums.  `bias` [outs] float32
-// or null (never with `gated`).
+// or null; with `gated`, `clamp` in its place.
 extern "C" int akv_linear_packed_normed(const float* stream_in, const void* delta, const float* norm_weight, float eps,
                                         float* stream_out, const void* wp, void* y, int rows, int outs, int k,
                                         int n_tiles, int k_tiles, int gated, const float* bias, hipStream_t stream) {

@@ -405,7 +405,7 @@ __global__ __launch_bounds__((A * kHalves + kFetchers) * 64) void linear_mid_ker
 #pragma unroll
       for (int mt = 0; mt < MT; ++mt)
         if (tile0 + rt < n_tiles)
-          store_tile<TY>(y, silu_times(acc[rt][mt], acc[rt + 1][mt]), row0 + mt * 16 + r, ((tile0 + rt) >> 1) * 16 + g * 4,
+          store_tile<TY>(y, gate_times(acc[rt][mt], acc[rt + 1][mt], bias), row0 + mt * 16 + r, ((tile0 + rt) >> 1) * 16 + g * 4,
                          rows, outs);
   } else {
 #pragma unroll
@@ -508,7 +508,7 @@ int launch_mid(const MidPlan& p, const void* x, const void* wp, void* y, float* 
   if (blocks > 0x7fffffffL) return -2;
   linear_mid_kernel<A, MT, RT, G, GATED, TY><<<static_cast<unsigned>(blocks), (A * kHalves + kFetchers) * 64, lds, stream>>>(
       static_cast<const bf16_t*>(x), static_cast<const uintx4*>(wp), static_cast<TY*>(y), partial, counters, rows, outs,
-      k, k_tiles, n_tiles, p.bands, p.parts, p.part_tiles, p.m_blocks, GATED ? nullptr : bias, fold);
+      k, k_tiles, n_tiles, p.bands, p.parts, p.part_tiles, p.m_blocks, bias, fold);
   return AKV_LAUNCH_STATUS();
 }
 
@@ -549,8 +549,8 @@ extern "C" int akv_linear_mid_workspace(int rows, int n_tiles, int k_tiles, int 
 // akv_linear_packed_swiglu).  `along` (waves along a band: 2..4), `rt` (row tiles per wave, 1 or 2), `depth`
 // (register sets of the weight ring: 2 with rt = 2, 4 with rt = 1) and `parts` (blocks along k, a power of two) may be 0: chosen here.
 // `partial_floats` and `counter_words` say how much `partial` and `counters` hold: a cut that needs more
-// (akv_linear_mid_workspace tells) is refused with -3 and nothing is launched.  `bias` [outs] float32 or null (never with
-// `gated`): added to the float32 sums before they are rounded.
+// (akv_linear_mid_workspace tells) is refused with -3 and nothing is launched.  `bias` [outs] float32 or null:
+// added to the float32 sums before they are rounded; with `gated`, `clamp` in its place (akv_linear_packed_swiglu).
 namespace {
 int linear_mid(const void* x, const void* wp, void* y, int y_dtype, float* partial, long partial_floats,
                unsigned* counters, long counter_words, int rows, int outs, int k, int n_tiles, int k_tiles, int gated,
@@ -558,7 +558,6 @@ int linear_mid(const void* x, const void* wp, void* y, int y_dtype, float* parti
   if (rows <= 0 || outs <= 0) return 0;
   if ((k & 7) != 0 || k_tiles * 32 < k) return -2;
   if (gated ? ((outs & 15) != 0 || n_tiles * 8 != outs) : n_tiles * 16 < outs) return -2;
-  if (gated && bias != nullptr) return -2;
   if (along < 0 || along == 1 || along > 4 || rt < 0 || rt > 2 || depth < 0 || parts < 0 || (parts & (parts - 1)) != 0) return -2;
   const MidPlan p = plan_mid(rows, n_tiles, k_tiles, gated != 0, along, rt, depth, parts);
   if (p.along == 0) return -2;
@@ -609,7 +608,7 @@ extern "C" int akv_linear_mid_adds(const void* x, const void* wp, void* y, float
 }
 
 // The product that reads rows left by akv_linear_mid_adds: y = (x W^T) * rsqrt(sum of squares of the row / k + eps) (+
-// bias; gated: silu of the scaled gate times the scaled up), the row's sum added up from sums_in [groups][sum_stride].
+// bias; gated: what `gate_times` makes of the scaled gate and the scaled up, `bias` being its `clamp`), the row's sum added up from sums_in [groups][sum_stride].
 // Refused with -2 where `groups` exceeds akv_linear_mid_most_groups(rows).
 extern "C" int akv_linear_mid_rowscaled(const void* x, const void* wp, void* y, int y_dtype, float* partial,
                                         long partial_floats, unsigned* counters, long counter_words, int rows, int outs,

@@ -65,10 +65,22 @@ __device__ __forceinline__ floatx4 plus_bias(floatx4 acc, const float* __restric
   return acc;
 }
 
-__device__ __forceinline__ floatx4 silu_times(floatx4 gate, floatx4 up) {
+// What a gated product stores.  `clamp` null: silu(gate) * up.  Otherwise its three numbers are a limit, a slope and a
+// shift: with g = min(gate, limit) and u = the up value held to [-limit, limit], g * sigmoid(slope g) * (u + shift).
+__device__ __forceinline__ floatx4 gate_times(floatx4 gate, floatx4 up, const float* __restrict__ clamp) {
   floatx4 v;
+  float slope = 1.f;
+  if (clamp != nullptr) {
+    const float limit = clamp[0], shift = clamp[2];
+    slope = clamp[1];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) v[i] = gate[i] / (1.f + expf(-gate[i])) * up[i];
+    for (int i = 0; i < 4; ++i) {
+      gate[i] = fminf(gate[i], limit);
+      up[i] = fminf(fmaxf(up[i], -limit), limit) + shift;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = gate[i] / (1.f + expf(-slope * gate[i])) * up[i];
   return v;
 }
 

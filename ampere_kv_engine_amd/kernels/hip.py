@@ -62,10 +62,14 @@ class PackedWeight:
 class GatedWeight:
     """Gate and up matrices [inter, k] of a gated feed-forward as ONE packed matrix whose row tiles alternate:
     tile 2t holds gate rows 16t .. 16t + 15, tile 2t + 1 the up rows of the same features; the packing is `paired`,
-    so the wave that owns both reads them as one run."""
+    so the wave that owns both reads them as one run.  `clamp` = (limit, slope, shift) makes it the clamped gate -
+    g * sigmoid(slope * g) * (u + shift) with g = min(gate, limit), u the up value held to [-limit, limit] - instead of
+    silu(gate) * up."""
 
-    def __init__(self, gate: torch.Tensor, up: torch.Tensor, keep_row_major: bool = False):
+    def __init__(self, gate: torch.Tensor, up: torch.Tensor, keep_row_major: bool = False, clamp=None):
         inter, k = gate.shape
+        self.clamp = tuple(float(number) for number in clamp) if clamp is not None else None
+        self.clamp_numbers = torch.tensor(self.clamp, dtype=torch.float32, device=gate.device) if clamp is not None else None
         self.inter, self.k = inter, k
         # what a library product reads: gate rows, then up rows
         self.stacked = torch.cat((gate, up), dim=0).contiguous() if keep_row_major else None
@@ -629,8 +633,8 @@ class HipKernels(PartsKernels, KernelSet):
         return self._route("linear", packed.outs, packed.k, rows, packed.row_major is not None, dtype) == "mid"
 
     def linear_rowscaled(self, x, sums, eps, weight, out, bias=None, row_tiles: int = 0) -> None:
-        """out = (x W^T) with every row divided by sqrt(mean of squares + eps), plus `bias` (a `GatedWeight`: silu of
-        the scaled gate times the scaled up): x [rows, k] are rows that `add_to_stream` left - the residual sum times
+        """out = (x W^T) with every row divided by sqrt(mean of squares + eps), plus `bias` (a `GatedWeight`: its
+        gate of the scaled gate and up): x [rows, k] are rows that `add_to_stream` left - the residual sum times
         the norm's weight -, sums [groups, rows rounded up to 16] the partial sums of squares of the residual rows."""
         gated = isinstance(weight, GatedWeight)
         packed = weight.packed if gated else weight
@@ -639,9 +643,7 @@ class HipKernels(PartsKernels, KernelSet):
         self._dense(x, "x", torch.bfloat16, (rows, packed.k))
         self._dense(out, "out", torch.bfloat16, (rows, outs))
         self._dense(packed.data, "packed weight", torch.bfloat16)
-        if bias is not None and gated:
-            raise KernelError("the gated product takes no bias")
-        self._bias(bias, outs)
+        bias = self._bias_or_clamp(weight, bias, outs)
         if rows <= self.FOLD_NORM_ROWS:         # a decode step: sums per (16 values of a row, row), as `linear_adds` leaves them
             self._dense(sums, "sums", torch.float32, ((packed.k + 15) // 16, 16))
             pieces, arrivals = self._exchange(packed.n_tiles)
@@ -702,9 +704,7 @@ class HipKernels(PartsKernels, KernelSet):
         outs = weight.inter if gated else packed.outs
         self._dense(out, "out", torch.bfloat16, (rows, outs))
         self._dense(packed.data, "packed weight", torch.bfloat16)
-        if bias is not None and gated:
-            raise KernelError("the gated product takes no bias")
-        self._bias(bias, outs)
+        bias = self._bias_or_clamp(weight, bias, outs)
         pieces, arrivals = self._exchange(packed.n_tiles)
         self._check(self.lib.akv_linear_scaled(_ptr(stream), _ptr(sums), (k + 15) // 16, _ptr(norm_weight),
                                                ctypes.c_float(eps), _ptr(packed.data), _ptr(out), _ptr(pieces),
@@ -769,14 +769,23 @@ class HipKernels(PartsKernels, KernelSet):
         self._check(self.lib.akv_linear_packed_normed(
             _ptr(stream), _ptr(delta), _ptr(norm_weight), ctypes.c_float(eps), _ptr(stream_out), _ptr(packed.data),
             _ptr(out), rows, outs, k, packed.n_tiles, packed.k_tiles, 1 if gated else 0,
-            _ptr(self._bias(bias, outs) if not gated else None), self._stream()), "linear_after_norm")
+            _ptr(self._bias_or_clamp(weight, bias, outs)), self._stream()), "linear_after_norm")
 
-    def prepare_gated_linear(self, gate: torch.Tensor, up: torch.Tensor):
+    def _bias_or_clamp(self, weight, bias, outs: int):
+        """What a product's kernel gets as its `bias`: the bias, or the numbers of a clamped gate."""
+        if not isinstance(weight, GatedWeight):
+            return self._bias(bias, outs)
+        if bias is not None:
+            raise KernelError("the gated product takes no bias")
+        return weight.clamp_numbers
+
+    def prepare_gated_linear(self, gate: torch.Tensor, up: torch.Tensor, clamp=None):
         """The packing for `gated_linear`, or None where the two matrices have to stay a stacked product followed by
-        `swiglu` (float32 weights, sizes the packed kernels do not take)."""
+        an activation kernel (float32 weights, sizes the packed kernels do not take).  `clamp` = (limit, slope, shift):
+        the clamped gate instead of silu."""
         if (gate.dtype == torch.bfloat16 and up.dtype == torch.bfloat16 and gate.shape == up.shape
                 and gate.shape[1] % 8 == 0 and gate.shape[0] % 16 == 0):
-            weight = GatedWeight(gate, up, keep_row_major=self.library_products_above is not None)
+            weight = GatedWeight(gate, up, keep_row_major=self.library_products_above is not None, clamp=clamp)
             self._products.setdefault(("gated", weight.inter, weight.k), weight)
             self._reserve_exchange(weight.packed.n_tiles)
             return weight
@@ -790,7 +799,7 @@ class HipKernels(PartsKernels, KernelSet):
         return (rows, 2 * weight.inter) if wanted else None
 
     def gated_linear(self, x, weight: GatedWeight, out, scratch=None):
-        """out [rows, inter] = silu(x Wgate^T) * (x Wup^T): one kernel, from float32 accumulators; where the library
+        """out [rows, inter] = silu(x Wgate^T) * (x Wup^T), or the clamped gate of the weight's `clamp`: one kernel, from float32 accumulators; where the library
         takes the product, its stacked product into `scratch`, then the activation kernel."""
         rows = x.shape[0]
         packed = weight.packed
@@ -805,14 +814,17 @@ class HipKernels(PartsKernels, KernelSet):
                                   "buffer that gated_scratch() describes")
             self._dense(scratch, "scratch", torch.bfloat16, (rows, 2 * weight.inter))
             torch.mm(x, weight.stacked.t(), out=scratch)
-            self.swiglu(scratch, out)
+            if weight.clamp is None:
+                self.swiglu(scratch, out)
+            else:
+                self.gated_activation(scratch, out, "clamped", *weight.clamp)
         elif route == "mid":
-            self._mid(x, packed, out, rows, weight.inter, True)
+            self._mid(x, packed, out, rows, weight.inter, True, weight.clamp_numbers)
         else:
             operand, packed_rows = self._operand_rows(x, rows, weight.k)
             self._check(self.lib.akv_linear_packed_swiglu(_ptr(operand), _ptr(packed.data), _ptr(out), _code(out), rows,
                                                           weight.inter, weight.k, packed.n_tiles, packed.k_tiles,
-                                                          packed_rows, self._stream()), "gated_linear")
+                                                          packed_rows, _ptr(weight.clamp_numbers), self._stream()), "gated_linear")
 
     def swiglu(self, gate_up, out):
         tokens, inter = out.shape

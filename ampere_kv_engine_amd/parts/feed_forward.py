@@ -3,7 +3,8 @@ down( silu(x Wg^T) * (x Wu^T) ), silu on the gate only.  Gate and up are one pro
 also applies the activation before anything is stored (`gated_linear`); otherwise the stacked product is followed
 by the `swiglu` kernel.  With `activation="gelu_tanh"` the gate passes the tanh form of gelu instead of silu: the stacked
 product, then the activation kernel that takes either (`gated_activation`).  With `activation="clamped"` (`limit`, `slope`,
-`shift`): g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(slope * g) * (u + shift), by the same kernel."""
+`shift`): g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(slope * g) * (u + shift), by the one-pass product
+where there is one, else by that kernel."""
 
 from __future__ import annotations
 
@@ -43,8 +44,9 @@ class SwiGLU(Part):
 
     def load(self, fetch, prefix):
         gate, up = (fetch(spec) for spec in self.gate_up.tensors(self._prefix(prefix)))
-        self.gated = (self.rt.kernels.prepare_gated_linear(gate.contiguous(), up.contiguous())
-                      if self.activation == "silu" else None)        # (the one-pass product's epilogue is silu)
+        clamp = tuple(self.constants[name] for name in ("limit", "slope", "shift")) if self.constants else None
+        self.gated = (self.rt.kernels.prepare_gated_linear(gate.contiguous(), up.contiguous(), **({"clamp": clamp} if clamp else {}))
+                      if self.activation in ("silu", "clamped") else None)     # (what the one-pass product's epilogue can do)
         if self.gated is None:
             self.gate_up.adopt(torch.cat((gate, up), dim=0).contiguous())
         else:

@@ -916,6 +916,85 @@ def test_decode_products_leave_rows_for_a_product_that_scales_its_sums(hip, ref,
     assert torch.equal(got, again)
 
 
+CLAMP = (0.7, 1.702, 1.25)      # limit, slope, shift: about a third of the values below reach the limit
+
+
+def clamped(gate, up):
+    limit, slope, shift = CLAMP
+    gate, up = gate.clamp(max=limit), up.clamp(-limit, limit)
+    return gate * torch.sigmoid(slope * gate) * (up + shift)
+
+
+@pytest.mark.parametrize("rows", [1, 5, 16, 17, 40, 64, 130, 300])
+@pytest.mark.parametrize("inter,k", [(208, 264), (512, 1032)])
+def test_gated_product_with_a_clamped_gate(hip_own, hip_library, rows, inter, k):
+    """Every kernel that may take the product: the decode and skinny ones, the wide one, the mid-size one with several
+    cuts, the library's product followed by the activation kernel."""
+    import ctypes
+    from ampere_kv_engine_amd.kernels.hip import _ptr
+    gate, up = (rand(inter, k, dtype=torch.bfloat16, seed=601 + i, scale=0.05) for i in range(2))
+    x = rand(rows, k, dtype=torch.bfloat16, seed=603)
+    g, u = x.float() @ gate.float().T, x.float() @ up.float().T
+    want = clamped(g, u).bfloat16().float()
+    for kernels in (hip_own, hip_library):
+        weight = kernels.prepare_gated_linear(gate.cuda(), up.cuda(), CLAMP)
+        shape = kernels.gated_scratch(weight, rows, torch.bfloat16)
+        scratch = torch.empty(shape, dtype=torch.bfloat16, device="cuda") if shape else None
+        got = torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+        kernels.gated_linear(x.cuda(), weight, got, scratch)
+        reference = clamped(g.bfloat16().float(), u.bfloat16().float()).bfloat16().float() if shape else want
+        torch.testing.assert_close(got.cpu().float(), reference, rtol=1.6e-2, atol=2e-2 if shape else 1e-3)
+    if rows > 16:
+        partial = torch.empty(8 << 20, dtype=torch.float32, device="cuda")
+        counters = torch.zeros(4096, dtype=torch.int32, device="cuda")
+        stream = ctypes.c_void_p(torch.cuda.current_stream().cuda_stream)
+        xd = x.cuda()
+        for along, parts in ((0, 0), (2, 1), (4, 4)):
+            got = torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+            assert hip_own.lib.akv_linear_mid(
+                _ptr(xd), _ptr(weight.packed.data), _ptr(got), 1, _ptr(partial), ctypes.c_long(partial.numel()), _ptr(counters),
+                ctypes.c_long(counters.numel()), rows, inter, k, weight.packed.n_tiles, weight.packed.k_tiles, 1, along, 2, 2, parts,
+                _ptr(weight.clamp_numbers), stream) == 0
+            torch.testing.assert_close(got.cpu().float(), want, **tol(torch.bfloat16))
+
+
+@pytest.mark.parametrize("rows", [1, 3, 16, 40])
+def test_products_with_a_clamped_gate_that_norm_or_scale_their_rows(hip_own, ref, rows, monkeypatch):
+    monkeypatch.setattr(hip_own, "fold_norms", True)
+    monkeypatch.setattr(hip_own, "FOLD_NORM_ROWS", 16)
+    monkeypatch.setattr(hip_own, "NORM_IN_PRODUCT_ROWS", 4)
+    inter, k, eps = 208, 264, 1e-6
+    stream, delta = rand(rows, k, seed=611, scale=2.0), rand(rows, k, dtype=torch.bfloat16, seed=612)
+    gain = 1 + rand(k, seed=613, scale=0.1)
+    gate, up = (rand(inter, k, dtype=torch.bfloat16, seed=614 + i, scale=0.05) for i in range(2))
+    weight = hip_own.prepare_gated_linear(gate.cuda(), up.cuda(), CLAMP)
+    if rows <= 4:                       # the rows normed by the product's blocks
+        summed, normed = stream.clone(), torch.empty(rows, k, dtype=torch.bfloat16)
+        ref.add_rmsnorm(summed, delta, gain, eps, normed)
+        new, got = torch.empty(rows, k, device="cuda"), torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+        hip_own.linear_after_norm(stream.cuda(), delta.cuda(), gain.cuda(), eps, new, weight, got)
+        want = clamped(normed.float() @ gate.float().T, normed.float() @ up.float().T)
+        torch.testing.assert_close(got.cpu().float(), want.bfloat16().float(), **tol(torch.bfloat16))
+    padded = torch.zeros(rows, (k + 15) // 16 * 16)
+    padded[:, :k] = stream
+    by_tile = padded.pow(2).reshape(rows, -1, 16).sum(-1).T
+    sums = torch.zeros((k + 15) // 16, (rows + 15) // 16 * 16)
+    sums[:, :rows] = by_tile
+    if rows <= 16:                      # the rows normed from their sums of squares
+        normed = torch.empty(rows, k, dtype=torch.bfloat16)
+        ref.add_rmsnorm(stream.clone(), None, gain, eps, normed)
+        got = torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+        hip_own.linear_scaled(stream.cuda(), sums.cuda(), gain.cuda(), eps, weight, got)
+        want = clamped(normed.float() @ gate.float().T, normed.float() @ up.float().T)
+        assert_close_but_for_flipped_roundings(got, want.bfloat16())
+    left = (stream * gain).bfloat16()   # rows whose products are divided by their root mean square
+    scale = torch.rsqrt(stream.pow(2).mean(-1, keepdim=True) + eps)
+    got = torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+    hip_own.linear_rowscaled(left.cuda(), sums.cuda(), eps, weight, got)
+    want = clamped(left.float() @ gate.float().T * scale, left.float() @ up.float().T * scale)
+    torch.testing.assert_close(got.cpu().float(), want.bfloat16().float(), **tol(torch.bfloat16))
+
+
 def test_linear_keeps_other_weights_row_major(hip):
     assert isinstance(hip.prepare_linear(torch.zeros(4, 12, dtype=torch.bfloat16, device="cuda")), torch.Tensor)   # k % 8
     assert isinstance(hip.prepare_linear(torch.zeros(4, 16, device="cuda")), torch.Tensor)                         # float32

@@ -87,8 +87,8 @@ class TorchKernels(KernelSet):
         y = x.float() @ weight.float().T
         out.copy_((y if bias is None else y + bias.float()).to(out.dtype))
 
-    def prepare_gated_linear(self, gate, up):
-        return (gate, up)
+    def prepare_gated_linear(self, gate, up, clamp=None):
+        return (gate, up) if clamp is None else (gate, up, clamp)
 
     # ---- the residual sum and the norm inside the products (decode steps) -------------------------------
     def folds_norm(self, rows, hidden, dtype):
@@ -165,6 +165,11 @@ class TorchKernels(KernelSet):
 
     def gated_linear(self, x, weight, out, scratch=None):
         g, u = x.float() @ weight[0].float().T, x.float() @ weight[1].float().T
+        if len(weight) == 3:
+            limit, slope, shift = weight[2]
+            g, u = g.clamp(max=limit), u.clamp(-limit, limit) + shift
+            out.copy_((g * torch.sigmoid(slope * g) * u).to(out.dtype))
+            return
         out.copy_((g * torch.sigmoid(g) * u).to(out.dtype))
 
     def swiglu(self, gate_up, out):
