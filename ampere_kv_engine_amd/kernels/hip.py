@@ -346,6 +346,9 @@ class HipKernels(PartsKernels, KernelSet):
             return (rows + 15) // 16
         return 8 if rows <= 128 else 16 if rows <= 256 else 32 if rows <= 512 else None
 
+    NARROW_OUTS = 256
+    NARROW_K = 1024
+
     def _route(self, kind: str, outs: int, k: int, rows: int, has_row_major: bool, out_dtype) -> str:
         """Which kernel takes a bfloat16 product of more than 16 rows: "own" (the skinny kernel up to 64 rows, the
         wide one above), "mid" (17..512 rows: the block's waves share the activations through LDS) or "library".
@@ -358,12 +361,16 @@ class HipKernels(PartsKernels, KernelSet):
         there); the gated product up to 64 rows, and up to 128 where the two matrices hold no more than 64 M elements
         (Qwen3-8B: 47 against 57 us with the library's activation pass; Qwen3-14B: 100 / 101; Qwen3-32B: 126 / 112).
         Beyond, the library.  Without the library: the mid-size kernel up to 512 rows (it is faster than the skinny
-        one from 17 rows on), the wide one beyond."""
+        one from 17 rows on), the wide one beyond - except for a few outputs over a long k (`NARROW_OUTS`,
+        `NARROW_K`), of which the wide kernel makes a block per 128 rows: there the mid-size one, which cuts k over blocks
+        (16 to 256 outputs of 2,048 rows over k = 2,048: 11 to 16 us against 27 to 31; over 4,096: 14 to 19 against 50 to 54)."""
         library = (has_row_major and self.library_products_above is not None and rows > self.library_products_above
                    and out_dtype == torch.bfloat16)
         bucket = self._row_bucket(rows)
         if bucket is None:
-            return "library" if library else "own"
+            if library:
+                return "library"
+            return "mid" if kind == "linear" and outs <= self.NARROW_OUTS and k >= self.NARROW_K else "own"
         choice = self.product_choices.get((kind, outs, k, bucket))
         if choice == "library" and not library:
             choice = None

@@ -995,6 +995,20 @@ def test_products_with_a_clamped_gate_that_norm_or_scale_their_rows(hip_own, ref
     torch.testing.assert_close(got.cpu().float(), want.bfloat16().float(), **tol(torch.bfloat16))
 
 
+@pytest.mark.parametrize("rows,outs,k", [(513, 16, 1024), (700, 40, 1032), (2048, 64, 2048), (1030, 256, 4096), (900, 5, 1096)])
+def test_few_outputs_of_many_rows(hip, ref, rows, outs, k):
+    """Float32 results of a few features over a long k: the mid-size kernel takes them, whatever the number of rows."""
+    x, w = rand(rows, k, dtype=torch.bfloat16, seed=621), rand(outs, k, dtype=torch.bfloat16, seed=622, scale=0.05)
+    bias = rand(outs, seed=623)
+    packed = hip.prepare_linear(w.cuda())
+    assert hip._route("linear", outs, k, rows, packed.row_major is not None, torch.float32) == "mid"
+    for b in (None, bias):
+        got = torch.full((rows, outs), float("nan"), device="cuda")
+        hip.linear(x.cuda(), packed, got, b.cuda() if b is not None else None)
+        want = x.float() @ w.float().T + (b if b is not None else 0.0)
+        torch.testing.assert_close(got.cpu(), want, rtol=1e-4, atol=1e-4)
+
+
 def test_linear_keeps_other_weights_row_major(hip):
     assert isinstance(hip.prepare_linear(torch.zeros(4, 12, dtype=torch.bfloat16, device="cuda")), torch.Tensor)   # k % 8
     assert isinstance(hip.prepare_linear(torch.zeros(4, 16, device="cuda")), torch.Tensor)                         # float32
