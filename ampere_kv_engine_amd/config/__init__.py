@@ -5,9 +5,11 @@ from .tukevik import TukevikConfig
 from .lirulix import LirulixConfig
 from .mekuvik import MekuvikConfig
 from .bolatar import BolatarConfig
+from .ziferax import ZiferaxConfig
 from .registry import architecture_of, known_architectures, load_config, register_architecture
 from .engine import EngineConfig
 
 __all__ = ["LayerSpec", "ModelSpec", "PartSpec", "RunEntry", "default_run_order", "part", "ConfigError",
-           "Qwen3Config", "KeranexConfig", "TukevikConfig", "LirulixConfig", "MekuvikConfig", "BolatarConfig", "architecture_of", "known_architectures", "load_config", "register_architecture",
+           "Qwen3Config", "KeranexConfig", "TukevikConfig", "LirulixConfig", "MekuvikConfig", "BolatarConfig", "ZiferaxConfig",
+           "architecture_of", "known_architectures", "load_config", "register_architecture",
            "EngineConfig"]

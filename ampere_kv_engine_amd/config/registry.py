@@ -18,6 +18,7 @@ from .lirulix import LirulixConfig
 from .mekuvik import MekuvikConfig
 from .qwen3 import ConfigError, Qwen3Config
 from .tukevik import TukevikConfig
+from .ziferax import ZiferaxConfig
 from .specs import ModelSpec
 
 
@@ -71,3 +72,4 @@ register_architecture(TukevikConfig.architecture, TukevikConfig)
 register_architecture(LirulixConfig.architecture, LirulixConfig)
 register_architecture(MekuvikConfig.architecture, MekuvikConfig)
 register_architecture(BolatarConfig.architecture, BolatarConfig)
+register_architecture(ZiferaxConfig.architecture, ZiferaxConfig)

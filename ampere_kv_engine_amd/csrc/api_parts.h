@@ -22,11 +22,15 @@ int akv_note_fed_tokens(const int* ids, const int* q_start, const int* seq_slots
 // branch.  With `out` (dtype): out = stream / rms(stream) * pre_weight, rounded once.  With `delta2` (dtype; only beside a
 // `delta` that is not normed): stream += delta_scale * (delta + delta2) - two branches that read the same input; with
 // `post_weight2` both are normed first: stream += delta_scale * (delta / rms(delta) * post_weight + delta2 / rms(delta2) *
-// post_weight2), post_eps inside both roots.
+// post_weight2), post_eps inside both roots.  With `share` (dtype; beside branches that are not normed):
+// stream += delta_scale * (delta (+ delta2) + share_weights[t * share_stride] * share[t]).
 int akv_norm_add_norm(float* stream_buf, const void* delta, const float* post_weight, float post_eps,
                       const float* pre_weight, float pre_eps, void* out, int dtype, int tokens, int hidden,
                       float delta_scale, const float* offset, const void* delta2, const float* post_weight2,
-                      hipStream_t stream);
+                      const void* share, const float* share_weights, long share_stride, hipStream_t stream);
+// out[t] += weights[t * stride] * rows[t], both [tokens, hidden] of `dtype`, weights float32
+int akv_add_weighted_rows(const void* rows, const float* weights, long stride, void* out, int dtype, long tokens, int hidden,
+                          hipStream_t stream);
 // out[n] = table[id] (with `accumulate`: out[n] += table[id]), float32; an id of -1: the token chosen last for the row's
 // request, where the slot words are given.  The row is multiplied by `scale`; with `places` [place_rows, hidden] (`dtype`) the
 // row of the token's position is added (a position beyond the table poisons the row).
@@ -72,12 +76,13 @@ int akv_scaled_sum(const void* a, float scale_a, const void* b, float scale_b, v
 // square is taken over all query vectors of the token at once, and over all its key vectors.  `q_weight` [q_heads x maps x
 // dim], `k_weight` [kv_heads x maps x dim] (float32, may be null): multiplied in after the norm, before the rotation.
 // `value_eps` >= 0: value heads are divided by their root mean square (value_eps inside the root).  `temp_every` > 0: queries
-// at position p are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).
+// at position p are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).  `keyed_values`: the value heads are the
+// key heads as they were projected (vdim = dim, one map); rows hold no columns for values.
 int akv_unit_norm_write(const void* projected, long stride, int dtype, long tokens, int q_heads, int kv_heads, int dim,
                         int vdim, float eps, int normed, const int* slot_map, void* k_pages, void* v_pages, int page_size,
                         long num_pages, void* q_out, int maps, const float* table, int table_positions, int rot_dims,
                         const int* positions, const float* q_weight, const float* k_weight, int whole, int interleaved,
-                        float value_eps, float temp_coef, int temp_every, hipStream_t stream);
+                        float value_eps, float temp_coef, int temp_every, int keyed_values, hipStream_t stream);
 // out [tokens, q_heads, vdim].  score = (q . k) * scale, then softcap * tanh(score / softcap) where softcap > 0; a query at
 // position p sees the keys j <= p with j > p - window (window > 0; the request's first `keep_first` keys stay visible
 // behind the window) and floor(j / chunk) = floor(p / chunk) (chunk > 0);
@@ -250,9 +255,17 @@ int akv_route_chosen(const float* logits, float* gates, int tokens, int experts,
 // 3: relu squared; e(c) = c / ff below experts * ff, else `experts`
 int akv_gate_activation(const void* up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
                         int columns, int scored, int kind, int inside, hipStream_t stream);
-// act[t, c] = gates[t, e(c)] * silu(gate_up[t, c]) * gate_up[t, columns + c]; e(c) = c / ff below experts * ff, else `experts`
-int akv_gate_silu_mul(const void* gate_up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
-                      int columns, int scored, hipStream_t stream);
+// logits [tokens, outputs] -> gates [tokens, scored]: scores = softmax over all outputs; the `top` outputs with the largest
+// scores + correction are chosen (equal ones: the lower index) and weighted by score / (sum of the chosen scores + 1e-20).
+// A gates' row: the first `experts` outputs' weights, 0 where not chosen; with `shared` a column of 1; with outputs > experts
+// a last column, the sum of the chosen weights of outputs `experts` on (identity experts).
+int akv_route_corrected(const float* logits, const float* correction, float* gates, int tokens, int experts, int outputs,
+                        int scored, int top, int shared, hipStream_t stream);
+// act[t, c] = gates[t, e(c)] * g * sigmoid(slope g) * (u + shift) with g = min(gate_up[t, c], limit) and u = gate_up[t, columns +
+// c] held to [-limit, limit]; e(c) = c / ff below experts * ff, else `experts`, where `shared_limit` stands for `limit`.
+// (Infinite limits, slope 1 and shift 0: silu(gate) * up.)
+int akv_gate_pair_mul(const void* gate_up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
+                      int columns, int scored, float limit, float shared_limit, float slope, float shift, hipStream_t stream);
 // act[t, e * ff + j] = gates[t, e] * relu(up[t, e * ff + j])^2
 int akv_gate_relu_squared(const void* up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
                           hipStream_t stream);

@@ -31,7 +31,8 @@ __device__ __forceinline__ void wave_sync_lds() {
 // its key vectors): every wave sums its side's whole projection for itself.  `q_weight` [q vectors x dim] and `k_weight`
 // [k vectors x dim] (float32, either may be null) multiply the normed values, before the rotation.  With `temp_every` > 0 a
 // query is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at its position p; with `value_eps` >= 0 a value
-// head is divided by its root mean square (value_eps inside the root) before it is written.
+// head is divided by its root mean square (value_eps inside the root) before it is written.  The value heads lie from column
+// `values_at` of a row on: behind the keys, or - values that are the keys as they were projected - where the keys lie.
 // One (token, item): `which` < q_vectors is a query vector, then the key vectors, then the value heads.  `given` > 0: the
 // factor 1 / rms of the item's side, formed by the caller over the whole projection; else the vector norms itself.
 template <typename T>
@@ -42,7 +43,7 @@ __device__ __forceinline__ void unit_norm_item(const T* __restrict__ row, long n
                                                const float* __restrict__ table, int table_positions, int rot_dims,
                                                const int* __restrict__ positions, const float* __restrict__ q_weight,
                                                const float* __restrict__ k_weight, int interleaved, float value_eps,
-                                               float temp_coef, int temp_every) {
+                                               float temp_coef, int temp_every, int values_at) {
   const int q_vectors = q_heads * maps, k_vectors = kv_heads * maps;
   if (which < q_vectors + k_vectors) {
     const bool is_q = which < q_vectors;
@@ -100,7 +101,7 @@ __device__ __forceinline__ void unit_norm_item(const T* __restrict__ row, long n
     const long slot = slot_map[n];
     const long page = slot / page_size;
     if (slot < 0 || page >= num_pages) return;
-    const T* x = row + static_cast<long>(q_vectors + k_vectors) * dim + static_cast<long>(h) * vdim;
+    const T* x = row + values_at + static_cast<long>(h) * vdim;
     T* y = v_pages + (page * kv_heads + h) * vdim * page_size + slot % page_size;
     if (value_eps >= 0.f) {      // values divided by their root mean square per head
       float squares = 0.f;
@@ -126,7 +127,7 @@ __global__ __launch_bounds__(256) void unit_norm_write_kernel(const T* __restric
                                                               int rot_dims, const int* __restrict__ positions,
                                                               const float* __restrict__ q_weight,
                                                               const float* __restrict__ k_weight, int interleaved,
-                                                              float value_eps, float temp_coef, int temp_every) {
+                                                              float value_eps, float temp_coef, int temp_every, int values_at) {
   const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   const int items = (q_heads + kv_heads) * maps + kv_heads;
   const long item = static_cast<long>(blockIdx.x) * waves + wave;
@@ -134,7 +135,7 @@ __global__ __launch_bounds__(256) void unit_norm_write_kernel(const T* __restric
   const long n = item / items;
   unit_norm_item<T>(projected + n * stride, n, static_cast<int>(item % items), lane, q_heads, kv_heads, dim, vdim, eps, normed,
                     0.f, slot_map, k_pages, v_pages, page_size, num_pages, q_out, maps, table, table_positions, rot_dims,
-                    positions, q_weight, k_weight, interleaved, value_eps, temp_coef, temp_every);
+                    positions, q_weight, k_weight, interleaved, value_eps, temp_coef, temp_every, values_at);
 }
 
 // The same with the root mean square taken over all of a token's query vectors at once, and over all its key vectors: a
@@ -149,7 +150,7 @@ __global__ __launch_bounds__(1024) void unit_norm_write_whole_kernel(const T* __
                                                                     int rot_dims, const int* __restrict__ positions,
                                                                     const float* __restrict__ q_weight,
                                                                     const float* __restrict__ k_weight, int interleaved,
-                                                                    float value_eps, float temp_coef, int temp_every) {
+                                                                    float value_eps, float temp_coef, int temp_every, int values_at) {
   __shared__ float scratch[16];
   const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   const long n = blockIdx.x;
@@ -167,7 +168,7 @@ __global__ __launch_bounds__(1024) void unit_norm_write_whole_kernel(const T* __
   for (int which = wave; which < items; which += waves)
     unit_norm_item<T>(row, n, which, lane, q_heads, kv_heads, dim, vdim, eps, 1, which < q_vectors ? q_scale : k_scale, slot_map,
                       k_pages, v_pages, page_size, num_pages, q_out, maps, table, table_positions, rot_dims, positions, q_weight,
-                      k_weight, interleaved, value_eps, temp_coef, temp_every);
+                      k_weight, interleaved, value_eps, temp_coef, temp_every, values_at);
 }
 
 constexpr int kMaxValueRegs = 4;  // value widths up to 256: each lane owns dims lane, lane + 64, ...
@@ -653,11 +654,13 @@ int akv_unit_norm_write(const void* projected, long stride, int dtype, long toke
                         int vdim, float eps, int normed, const int* slot_map, void* k_pages, void* v_pages, int page_size,
                         long num_pages, void* q_out, int maps, const float* table, int table_positions, int rot_dims,
                         const int* positions, const float* q_weight, const float* k_weight, int whole, int interleaved,
-                        float value_eps, float temp_coef, int temp_every, hipStream_t stream) {
+                        float value_eps, float temp_coef, int temp_every, int keyed_values, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (q_heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || page_size <= 0 || maps < 1) return -2;
   if (table != nullptr && (rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > dim || positions == nullptr)) return -2;
   if (temp_every > 0 && positions == nullptr) return -2;
+  if (keyed_values && (vdim != dim || maps != 1)) return -2;
+  const int values_at = keyed_values ? q_heads * dim : (q_heads + kv_heads) * maps * dim;
   const long items = tokens * ((q_heads + kv_heads) * maps + kv_heads);
   if (whole && normed) {
     // (few tokens: sixteen waves a token share its items; many: four, and the tokens fill the device)
@@ -666,14 +669,14 @@ int akv_unit_norm_write(const void* projected, long stride, int dtype, long toke
                                static_cast<const T*>(projected), stride, q_heads, kv_heads, dim, vdim, eps, slot_map,
                                static_cast<T*>(k_pages), static_cast<T*>(v_pages), page_size, num_pages, static_cast<T*>(q_out),
                                maps, table, table_positions, rot_dims, positions, q_weight, k_weight, interleaved, value_eps,
-                               temp_coef, temp_every));
+                               temp_coef, temp_every, values_at));
     return AKV_LAUNCH_STATUS();
   }
   AKV_DISPATCH(dtype, T, unit_norm_write_kernel<T><<<static_cast<unsigned>((items + 3) / 4), 256, 0, stream>>>(
                              static_cast<const T*>(projected), stride, tokens, q_heads, kv_heads, dim, vdim, eps, normed,
                              slot_map, static_cast<T*>(k_pages), static_cast<T*>(v_pages), page_size, num_pages,
                              static_cast<T*>(q_out), maps, table, table_positions, rot_dims, positions, q_weight,
-                             k_weight, interleaved, value_eps, temp_coef, temp_every));
+                             k_weight, interleaved, value_eps, temp_coef, temp_every, values_at));
   return AKV_LAUNCH_STATUS();
 }
 

@@ -1,5 +1,6 @@
 // A routed feed-forward's token-wise kernels: the choice of experts from the router's float32 logits (softmax over all
-// experts, the choice restricted to the best groups of neighbouring experts) and the experts' activation times the router's weight.
+// experts, the choice restricted to the best groups of neighbouring experts; over the chosen alone; sigmoids; a choice by
+// corrected scores) and the experts' activation times the router's weight.
 
 #include "common.h"
 #include "api_parts.h"
@@ -180,12 +181,94 @@ __global__ __launch_bounds__(256) void route_chosen_kernel(const float* __restri
   }
 }
 
-// act[t, c] = gates[t, e(c)] * silu(gate_up[t, c]) * gate_up[t, columns + c]: the experts' gate rows first, then their up
+// One wave per token: scores = softmax over all of the router's outputs; the `top` outputs with the largest score + correction
+// are chosen (equal ones: the lower index) and weighted by score / (the chosen scores' sum + 1e-20), a sum in the order of the
+// choice.  The first `experts` outputs are experts; the weights of chosen outputs beyond them - experts that return their input
+// - are added up into the row's last column.
+__global__ __launch_bounds__(256) void route_corrected_kernel(const float* __restrict__ logits,
+                                                              const float* __restrict__ correction, float* __restrict__ gates,
+                                                              int tokens, int experts, int outputs, int scored, int top,
+                                                              int shared) {
+  extern __shared__ float lds[];
+  const int waves = blockDim.x / kWave, wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
+  const int n = blockIdx.x * waves + wave;
+  if (n >= tokens) return;
+  float* score = lds + static_cast<size_t>(wave) * 2 * outputs;   // [outputs]
+  float* choice = score + outputs;                                // [outputs], -inf once chosen
+  const float* row = logits + static_cast<size_t>(n) * outputs;
+  float* gate_row = gates + static_cast<size_t>(n) * scored;
+  float highest = -INFINITY;
+  for (int e = lane; e < outputs; e += kWave) highest = fmaxf(highest, row[e]);
+  highest = wave_max(highest);
+  float total = 0.f;
+  for (int e = lane; e < outputs; e += kWave) {
+    const float raised = expf(row[e] - highest);
+    score[e] = raised;
+    total += raised;
+  }
+  total = wave_sum(total);
+  for (int e = lane; e < outputs; e += kWave) {       // (a lane reads back what it wrote itself)
+    const float s = score[e] / total;
+    score[e] = s;
+    choice[e] = s + correction[e];
+    if (e < experts) gate_row[e] = 0.f;
+  }
+  if (shared && lane == 0) gate_row[experts] = 1.f;
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  float sum = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < outputs; e += kWave) {
+      const float z = choice[e];
+      if (z > best) {            // (ascending e: the lower index keeps an equal one)
+        best = z;
+        at = e;
+      }
+    }
+#pragma unroll
+    for (int offset = kWave / 2; offset > 0; offset >>= 1) {
+      const float other = __shfl_xor(best, offset, kWave);
+      const int other_at = __shfl_xor(at, offset, kWave);
+      if (other > best || (other == best && other_at < at)) {
+        best = other;
+        at = other_at;
+      }
+    }
+    if (at == 0x7fffffff) break;      // (nothing finite left: cannot happen while top <= outputs and logits are finite; uniform)
+    sum += score[at];
+    if (lane == at % kWave) choice[at] = -INFINITY;       // (the lane that reads it)
+  }
+  float beyond = 0.f;
+  for (int e = lane; e < outputs; e += kWave) {
+    if (choice[e] != -INFINITY) continue;
+    const float weight = score[e] / (sum + 1e-20f);
+    if (e < experts) gate_row[e] = weight;
+    else beyond += weight;
+  }
+  if (outputs > experts) {
+    beyond = wave_sum(beyond);
+    if (lane == 0) gate_row[scored - 1] = beyond;
+  }
+}
+
+// What an expert with a gate makes of its two products: g sigmoid(slope g) (u + shift), g = min(gate, limit), u = up held to
+// [-limit, limit].  Infinite limits, slope 1 and shift 0 make it silu(gate) * up.  (Comparisons that keep a NaN.)
+__device__ __forceinline__ float gated_pair(float z, float u, float limit, float slope, float shift) {
+  z = z > limit ? limit : z;
+  u = u > limit ? limit : (u < -limit ? -limit : u);
+  return z / (1.f + expf(-slope * z)) * (u + shift);
+}
+
+// act[t, c] = gates[t, e(c)] * gated_pair(gate_up[t, c], gate_up[t, columns + c]): the experts' gate rows first, then their up
 // rows; column c belongs to expert c / ff while c < experts * ff and to the expert every token uses beyond (gate number
-// `experts`).  Float32 up to the one rounding; an expert that was not chosen gives exact zeros.
+// `experts`, with a limit of its own).  Float32 up to the one rounding; an expert that was not chosen gives exact zeros.
 template <typename T>
-__global__ void gate_silu_mul_kernel(const T* __restrict__ gate_up, const float* __restrict__ gates, T* __restrict__ act,
-                                     long tokens, int experts, int ff, int columns, int scored) {
+__global__ void gate_pair_mul_kernel(const T* __restrict__ gate_up, const float* __restrict__ gates, T* __restrict__ act,
+                                     long tokens, int experts, int ff, int columns, int scored, float limit,
+                                     float shared_limit, float slope, float shift) {
   const long index = static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (index >= tokens * columns) return;
   const long n = index / columns;
@@ -194,17 +277,17 @@ __global__ void gate_silu_mul_kernel(const T* __restrict__ gate_up, const float*
   const float g = gates[n * scored + e];
   float value = 0.f;
   if (g != 0.f) {
-    const float z = to_float(gate_up[n * 2 * columns + c]);
-    value = g * (z / (1.f + expf(-z)) * to_float(gate_up[n * 2 * columns + columns + c]));
+    value = g * gated_pair(to_float(gate_up[n * 2 * columns + c]), to_float(gate_up[n * 2 * columns + columns + c]),
+                           e < experts ? limit : shared_limit, slope, shift);
   }
   act[index] = from_float<T>(value);
 }
 
 // The same, eight values a thread (16 bytes of bfloat16 per load and store), where every expert's width and the shared
 // one's are multiples of 8: a thread's eight columns then belong to one expert.
-__global__ void gate_silu_mul_by8_kernel(const bf16_t* __restrict__ gate_up, const float* __restrict__ gates,
+__global__ void gate_pair_mul_by8_kernel(const bf16_t* __restrict__ gate_up, const float* __restrict__ gates,
                                          bf16_t* __restrict__ act, long tokens, int experts, int ff, int columns,
-                                         int scored) {
+                                         int scored, float limit, float shared_limit, float slope, float shift) {
   const long index = (static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x) * 8;
   if (index >= tokens * columns) return;
   const long n = index / columns;
@@ -213,6 +296,7 @@ __global__ void gate_silu_mul_by8_kernel(const bf16_t* __restrict__ gate_up, con
   const float g = gates[n * scored + e];
   uint4 packed = make_uint4(0u, 0u, 0u, 0u);
   if (g != 0.f) {
+    const float bound = e < experts ? limit : shared_limit;
     const uint4 zs = *reinterpret_cast<const uint4*>(gate_up + n * 2 * columns + c);
     const uint4 us = *reinterpret_cast<const uint4*>(gate_up + n * 2 * columns + columns + c);
     const uint32_t zw[4] = {zs.x, zs.y, zs.z, zs.w}, uw[4] = {us.x, us.y, us.z, us.w};
@@ -221,7 +305,7 @@ __global__ void gate_silu_mul_by8_kernel(const bf16_t* __restrict__ gate_up, con
     for (int k = 0; k < 4; ++k) {
       const float z0 = __uint_as_float(zw[k] << 16), z1 = __uint_as_float(zw[k] & 0xffff0000u);
       const float u0 = __uint_as_float(uw[k] << 16), u1 = __uint_as_float(uw[k] & 0xffff0000u);
-      outs[k] = bf16_pair(g * (z0 / (1.f + expf(-z0)) * u0), g * (z1 / (1.f + expf(-z1)) * u1));
+      outs[k] = bf16_pair(g * gated_pair(z0, u0, bound, slope, shift), g * gated_pair(z1, u1, bound, slope, shift));
     }
     packed = make_uint4(outs[0], outs[1], outs[2], outs[3]);
   }
@@ -316,20 +400,34 @@ int akv_route_chosen(const float* logits, float* gates, int tokens, int experts,
   return AKV_LAUNCH_STATUS();
 }
 
-int akv_gate_silu_mul(const void* gate_up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
-                      int columns, int scored, hipStream_t stream) {
+int akv_route_corrected(const float* logits, const float* correction, float* gates, int tokens, int experts, int outputs,
+                        int scored, int top, int shared, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  if (experts <= 0 || outputs < experts || top <= 0 || top > outputs || correction == nullptr) return -2;
+  if (scored != experts + (shared ? 1 : 0) + (outputs > experts ? 1 : 0)) return -2;
+  const int waves = 4;
+  const size_t lds_bytes = static_cast<size_t>(waves) * 2 * outputs * 4;
+  if (lds_bytes > 64 * 1024) return -2;
+  route_corrected_kernel<<<(tokens + waves - 1) / waves, waves * kWave, lds_bytes, stream>>>(
+      logits, correction, gates, tokens, experts, outputs, scored, top, shared);
+  return AKV_LAUNCH_STATUS();
+}
+
+int akv_gate_pair_mul(const void* gate_up, const float* gates, void* act, int dtype, long tokens, int experts, int ff,
+                      int columns, int scored, float limit, float shared_limit, float slope, float shift, hipStream_t stream) {
   const long count = tokens * columns;
   if (count <= 0) return 0;
   if (columns < experts * ff || scored < experts + (columns > experts * ff ? 1 : 0)) return -2;
   if (dtype == kBF16 && ff % 8 == 0 && columns % 8 == 0 && reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(act) % 16 == 0) {
-    gate_silu_mul_by8_kernel<<<static_cast<unsigned>((count / 8 + 255) / 256), 256, 0, stream>>>(
-        static_cast<const bf16_t*>(gate_up), gates, static_cast<bf16_t*>(act), tokens, experts, ff, columns, scored);
+    gate_pair_mul_by8_kernel<<<static_cast<unsigned>((count / 8 + 255) / 256), 256, 0, stream>>>(
+        static_cast<const bf16_t*>(gate_up), gates, static_cast<bf16_t*>(act), tokens, experts, ff, columns, scored, limit,
+        shared_limit, slope, shift);
     return AKV_LAUNCH_STATUS();
   }
-  AKV_DISPATCH(dtype, T, gate_silu_mul_kernel<T><<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(
+  AKV_DISPATCH(dtype, T, gate_pair_mul_kernel<T><<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(
                              static_cast<const T*>(gate_up), gates, static_cast<T*>(act), tokens, experts, ff, columns,
-                             scored));
+                             scored, limit, shared_limit, slope, shift));
   return AKV_LAUNCH_STATUS();
 }
 

@@ -80,10 +80,13 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
                                                                  T* __restrict__ out, int hidden, float delta_scale,
                                                                  const float* __restrict__ offset,
                                                                  const T* __restrict__ delta2,
-                                                                 const float* __restrict__ post_weight2) {
+                                                                 const float* __restrict__ post_weight2,
+                                                                 const T* __restrict__ share,
+                                                                 const float* __restrict__ share_weights, long share_stride) {
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * hidden;
   float4 kept[GROUPS], added[GROUPS], second[GROUPS];
+  const float share_weight = share != nullptr ? share_weights[blockIdx.x * share_stride] : 0.f;
   // every load goes out before anything waits (a group beyond the row reads its last four values and counts for nothing)
 #pragma unroll
   for (int j = 0; j < GROUPS; ++j) {
@@ -94,6 +97,11 @@ __global__ __launch_bounds__(256) void norm_add_norm_rows_kernel(float* __restri
       second[j] = read4<T>(delta2 + base + i);
       if (post_weight2 == nullptr)
         added[j] = make_float4(added[j].x + second[j].x, added[j].y + second[j].y, added[j].z + second[j].z, added[j].w + second[j].w);
+    }
+    if (share != nullptr) {       // a share of what a branch read, weighted row by row
+      const float4 r = read4<T>(share + base + i);
+      added[j] = make_float4(fmaf(share_weight, r.x, added[j].x), fmaf(share_weight, r.y, added[j].y),
+                             fmaf(share_weight, r.z, added[j].z), fmaf(share_weight, r.w, added[j].w));
     }
   }
   float squares = 0.f;
@@ -168,7 +176,9 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(float* __restrict__ 
                                                             T* __restrict__ out, int hidden, float delta_scale,
                                                             const float* __restrict__ offset,
                                                             const T* __restrict__ delta2,
-                                                            const float* __restrict__ post_weight2) {
+                                                            const float* __restrict__ post_weight2,
+                                                            const T* __restrict__ share,
+                                                            const float* __restrict__ share_weights, long share_stride) {
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * hidden;
   float* s = stream + base;
@@ -198,7 +208,8 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(float* __restrict__ 
                                  to_float(delta2[base + i]) * second_scale * post_weight2[i]);
       } else
       for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-        const float both = delta2 != nullptr ? to_float(d[i]) + to_float(delta2[base + i]) : to_float(d[i]);
+        float both = delta2 != nullptr ? to_float(d[i]) + to_float(delta2[base + i]) : to_float(d[i]);
+        if (share != nullptr) both = fmaf(share_weights[blockIdx.x * share_stride], to_float(share[base + i]), both);
         s[i] += post_weight != nullptr ? both * post_scale * post_weight[i] : both * delta_scale;
       }
     }
@@ -378,6 +389,15 @@ __global__ __launch_bounds__(256) void norm_gate_rows4_kernel(const TX* __restri
     if (gate_act != 0) v = make_float4(v.x * gated(gate[j].x), v.y * gated(gate[j].y), v.z * gated(gate[j].z), v.w * gated(gate[j].w));
     write4<T>(out + n * out_stride + i, v);
   }
+}
+
+// ---- a share of one set of rows added to another: out[t] += weights[t * stride] * rows[t] ---------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void add_weighted_rows_kernel(const T* __restrict__ rows, const float* __restrict__ weights,
+                                                                long stride, T* __restrict__ out, long count, int hidden) {
+  const long index = static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x;
+  if (index >= count) return;
+  out[index] = from_float<T>(fmaf(weights[index / hidden * stride], to_float(rows[index]), to_float(out[index])));
 }
 
 // ---- a gated feed-forward's activation after a stacked product: out = act(gate) * up --------------------------------------
@@ -585,15 +605,26 @@ int akv_note_fed_tokens(const int* ids, const int* q_start, const int* seq_slots
   return AKV_LAUNCH_STATUS();
 }
 
+int akv_add_weighted_rows(const void* rows, const float* weights, long stride, void* out, int dtype, long tokens, int hidden,
+                          hipStream_t stream) {
+  const long count = tokens * hidden;
+  if (count <= 0) return 0;
+  if (stride < 1) return -2;
+  AKV_DISPATCH(dtype, T, add_weighted_rows_kernel<T><<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(
+                             static_cast<const T*>(rows), weights, stride, static_cast<T*>(out), count, hidden));
+  return AKV_LAUNCH_STATUS();
+}
+
 int akv_norm_add_norm(float* stream_buf, const void* delta, const float* post_weight, float post_eps,
                       const float* pre_weight, float pre_eps, void* out, int dtype, int tokens, int hidden,
                       float delta_scale, const float* offset, const void* delta2, const float* post_weight2,
-                      hipStream_t stream) {
+                      const void* share, const float* share_weights, long share_stride, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (out != nullptr && pre_weight == nullptr) return -2;
   if (delta2 != nullptr && (delta == nullptr || (post_weight != nullptr) != (post_weight2 != nullptr))) return -2;
   if (post_weight2 != nullptr && delta2 == nullptr) return -2;
-#define AKV_NORM_ARGS stream_buf, static_cast<const T*>(delta), post_weight, post_eps, pre_weight, pre_eps, static_cast<T*>(out), hidden, delta_scale, offset, static_cast<const T*>(delta2), post_weight2
+  if (share != nullptr && (delta == nullptr || post_weight != nullptr || share_weights == nullptr || share_stride < 0)) return -2;
+#define AKV_NORM_ARGS stream_buf, static_cast<const T*>(delta), post_weight, post_eps, pre_weight, pre_eps, static_cast<T*>(out), hidden, delta_scale, offset, static_cast<const T*>(delta2), post_weight2, static_cast<const T*>(share), share_weights, share_stride
   AKV_DISPATCH(dtype, T, {
     if (hidden % 4 == 0 && hidden >= 4 && hidden <= 256 * 4 * 2) norm_add_norm_rows_kernel<T, 2><<<tokens, 256, 0, stream>>>(AKV_NORM_ARGS);
     else if (hidden % 4 == 0 && hidden <= 256 * 4 * 8) norm_add_norm_rows_kernel<T, 8><<<tokens, 256, 0, stream>>>(AKV_NORM_ARGS);

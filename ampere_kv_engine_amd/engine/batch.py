@@ -128,6 +128,7 @@ class StepContext:
     fold_gain: object = None
     # set by a block around its mixer: the mixer may return an `Unsettled` instead of a tensor (`parts.base.NormedPair`)
     takes_unsettled_branch: bool = False
+    takes_input_share: bool = False         # set by a block around a branch that may return an `InputShare`
     # the device's persistent integer state (slot words, block tables) and what this step changes in it
     table_pages: int = 0                        # bound on the pages of the step's longest request (sizes launches)
     patches: torch.Tensor | None = None         # int32 [2 * patch_room]: (offset into slot_state, value) pairs

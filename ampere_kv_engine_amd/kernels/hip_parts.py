@@ -46,7 +46,7 @@ class PartsKernels:
                          "akv_conv_state_update", "akv_selective_scan", "akv_route", "akv_gate_relu_squared",
                          "akv_parts_slot_layout", "akv_conv_taps", "akv_scaled_sum", "akv_unit_norm_write",
                          "akv_gated_attention_rows", "akv_gated_attention_tiles", "akv_retention", "akv_retention_chunked", "akv_gated_linear_scan", "akv_route_chosen",
-                         "akv_gate_silu_mul", "akv_embed_normed", "akv_gated_activation", "akv_difference_norm_gate",
+                         "akv_gate_pair_mul", "akv_route_corrected", "akv_add_weighted_rows", "akv_embed_normed", "akv_gated_activation", "akv_difference_norm_gate",
                          "akv_delta_rule", "akv_embed_rows", "akv_norm_gate_rows", "akv_gate_activation", "akv_softcap",
                          "akv_token_shift", "akv_tanh_rows", "akv_time_mixing", "akv_matrix_memory"):
                 getattr(lib, name).restype = ctypes.c_int
@@ -106,13 +106,15 @@ class PartsKernels:
                                             self._stream()), "note_fed_tokens")
 
     def norm_add_norm(self, stream, delta, post_weight, post_eps, pre_weight, pre_eps, out, delta_scale: float = 1.0,
-                      offset=None, delta2=None, post_weight2=None) -> None:
+                      offset=None, delta2=None, post_weight2=None, share=None, share_weights=None, share_at: int = 0) -> None:
         """stream (float32) += delta / rms(delta) * post_weight (+= delta_scale * delta where `post_weight` is None; nothing
         where `delta` is None); then stream += offset (a float32 vector, the same on every row) where there is one; then,
         where `out` is given, out = stream / rms(stream) * pre_weight.  Float32 up to the one rounding of a stored result.
         `delta2` (beside a `delta` that is not normed): a second branch, stream += delta_scale * (delta + delta2).  With
         `post_weight2` both branches are normed: stream += delta_scale * (delta / rms(delta) * post_weight + delta2 /
-        rms(delta2) * post_weight2), with `post_eps` inside both roots."""
+        rms(delta2) * post_weight2), with `post_eps` inside both roots.  `share` (beside branches that are not normed): rows
+        of which a token's share is added to the branches before the scale, share_weights[t, share_at] * share[t]
+        (`share_weights` float32)."""
         tokens, hidden = stream.shape
         self._dense(stream, "stream", torch.float32)
         dtype = None
@@ -133,6 +135,12 @@ class PartsKernels:
             if delta2 is None:
                 self._refuse("a norm for a second branch without one")
             self._dense(post_weight2, "post_weight2", torch.float32, (hidden,))
+        share_stride = 0
+        if share is not None:
+            if delta is None or post_weight is not None:
+                self._refuse("a share of a branch's input comes beside branches that are not normed")
+            self._dense(share, "share", delta.dtype, (tokens, hidden))
+            share_stride = self._weight_column(share_weights, share_at, tokens)
         if offset is not None:
             self._dense(offset, "offset", torch.float32, (hidden,))
             dtype = dtype or torch.float32
@@ -141,8 +149,27 @@ class PartsKernels:
         self._check(self._parts().akv_norm_add_norm(_ptr(stream), _ptr(delta), _ptr(post_weight), ctypes.c_float(post_eps),
                                                     _ptr(pre_weight), ctypes.c_float(pre_eps), _ptr(out), _DTYPE_CODE[dtype],
                                                     tokens, hidden, ctypes.c_float(delta_scale), _ptr(offset), _ptr(delta2),
-                                                    _ptr(post_weight2), self._stream()),
+                                                    _ptr(post_weight2), _ptr(share),
+                                                    _ptr_at(share_weights, share_at) if share is not None else ctypes.c_void_p(0),
+                                                    _long(share_stride), self._stream()),
                     "norm_add_norm")
+
+    def _weight_column(self, weights, column: int, tokens: int) -> int:
+        """Checks a float32 column of weights, one a token; returns its stride."""
+        self._dense(weights, "weights", torch.float32)
+        if weights.dim() != 2 or weights.shape[0] != tokens or not 0 <= column < weights.shape[1]:
+            self._refuse(f"weights must be [{tokens}, more than {column}], got {tuple(weights.shape)}")
+        return weights.shape[1]
+
+    def add_weighted_rows(self, rows, weights, column: int, out) -> None:
+        """out[t] += weights[t, column] * rows[t]."""
+        tokens, hidden = out.shape
+        self._dense(out, "out")
+        self._dense(rows, "rows", out.dtype, (tokens, hidden))
+        stride = self._weight_column(weights, column, tokens)
+        self._check(self._parts().akv_add_weighted_rows(_ptr(rows), _ptr_at(weights, column), _long(stride), _ptr(out),
+                                                        self._code_of(out), _long(tokens), hidden, self._stream()),
+                    "add_weighted_rows")
 
     def embed_add(self, ids, table, out, ctx=None) -> None:
         """out[n] += table[id], float32: the embedding's rows added to a residual sum that already holds something.  With
@@ -709,6 +736,19 @@ class PartsKernels:
         self._check(self._parts().akv_route_chosen(_ptr(logits), _ptr(gates), tokens, experts, gates.shape[1], top,
                                                    1 if law == "sigmoid" else 0, self._stream()), "route_chosen")
 
+    def route_corrected(self, logits, correction, gates, experts: int, top: int, shared: bool) -> None:
+        """scores = softmax over all columns of `logits`; the `top` columns with the largest scores + `correction` are chosen
+        and weighted by their scores over the chosen scores' sum (+ 1e-20).  gates' columns: the first `experts` outputs'
+        weights (0 where not chosen); with `shared` a column of ones; with more outputs than experts a last column, the sum
+        of the weights of the chosen outputs beyond the experts."""
+        tokens, outputs = logits.shape
+        self._dense(logits, "logits", torch.float32)
+        self._dense(correction, "correction", torch.float32, (outputs,))
+        scored = experts + (1 if shared else 0) + (1 if outputs > experts else 0)
+        self._dense(gates, "gates", torch.float32, (tokens, scored))
+        self._check(self._parts().akv_route_corrected(_ptr(logits), _ptr(correction), _ptr(gates), tokens, experts, outputs,
+                                                      scored, top, 1 if shared else 0, self._stream()), "route_corrected")
+
     EXPERT_ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu_squared": 3}
 
     def gate_activation(self, up, gates, act, experts: int, ff: int, activation: str, inside: bool) -> None:
@@ -730,14 +770,25 @@ class PartsKernels:
     def gate_silu_mul(self, gate_up, gates, act, experts: int, ff: int) -> None:
         """act[t, c] = gates[t, e(c)] * silu(gate_up[t, c]) * gate_up[t, columns + c]; column c belongs to expert c // ff
         below experts * ff and to the expert every token uses beyond (gate number `experts`)."""
+        self._gate_pair_mul(gate_up, gates, act, experts, ff, float("inf"), float("inf"), 1.0, 0.0)
+
+    def gate_clamped_mul(self, gate_up, gates, act, experts: int, ff: int, limit: float, slope: float, shift: float,
+                         shared_limit: float) -> None:
+        """The same with the clamped gate in place of silu: g = min(gate, limit), u = up held to [-limit, limit],
+        gates * g sigmoid(slope g) (u + shift); `shared_limit` for the expert every token uses."""
+        self._gate_pair_mul(gate_up, gates, act, experts, ff, limit, shared_limit, slope, shift)
+
+    def _gate_pair_mul(self, gate_up, gates, act, experts, ff, limit, shared_limit, slope, shift) -> None:
         tokens, columns = act.shape
         self._dense(act, "act")
         self._dense(gate_up, "gate_up", act.dtype, (tokens, 2 * columns))
         self._dense(gates, "gates", torch.float32)
         if gates.dim() != 2 or gates.shape[0] != tokens or gates.shape[1] < experts + (1 if columns > experts * ff else 0):
             self._refuse(f"gates must be [tokens, at least the experts (and the shared one)], got {tuple(gates.shape)}")
-        self._check(self._parts().akv_gate_silu_mul(_ptr(gate_up), _ptr(gates), _ptr(act), self._code_of(act), _long(tokens),
-                                                    experts, ff, columns, gates.shape[1], self._stream()), "gate_silu_mul")
+        self._check(self._parts().akv_gate_pair_mul(
+            _ptr(gate_up), _ptr(gates), _ptr(act), self._code_of(act), _long(tokens), experts, ff, columns, gates.shape[1],
+            ctypes.c_float(limit), ctypes.c_float(shared_limit), ctypes.c_float(slope), ctypes.c_float(shift),
+            self._stream()), "gate_pair_mul")
 
     # ---- attention with unit-normed queries and keys, a softcap, chunks, a sink and a gate per head ----------------------
     MAX_VALUE_DIM = 256
@@ -759,7 +810,7 @@ class PartsKernels:
     def unit_norm_write(self, projected, q_heads, kv_heads, dim, vdim, eps, slot_map, k_pages, v_pages, q_out, at: int = 0,
                         maps: int = 1, table=None, rot_dims: int = 0, positions=None, q_weight=None, k_weight=None,
                         whole: bool = False, interleaved: bool = False, value_eps: float | None = None,
-                        temperature: tuple | None = None) -> None:
+                        temperature: tuple | None = None, keyed_values: bool = False) -> None:
         """projected [tokens, ... | q | k | v | ...] with q at column `at`: the query heads divided by their root mean square (eps inside the root;
         `eps` None: as they are) -> q_out; with `slot_map` the key heads, the same way, and the value heads into the
         tokens' slots of the pages.  `maps` > 1: a head's queries and keys are `maps` vectors of `dim` side by side, each
@@ -769,14 +820,18 @@ class PartsKernels:
         root mean square is taken over all of a token's query vectors at once, and over all its key vectors.  `q_weight`,
         `k_weight` (float32, one value per column of the queries and of the keys): multiplied in after the norm.
         `value_eps`: every value head is divided by its root mean square (value_eps inside the root) before it is written.
-        `temperature` (coef, every): a query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)."""
+        `temperature` (coef, every): a query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).
+        `keyed_values`: the value heads are the key heads as they were projected; the rows hold no columns for values."""
         tokens = projected.shape[0]
         if q_weight is not None:
             self._dense(q_weight, "q_weight", torch.float32, (q_heads * maps * dim,))
         if k_weight is not None:
             self._dense(k_weight, "k_weight", torch.float32, (kv_heads * maps * dim,))
         self._dense(projected, "projected")
-        if projected.dim() != 2 or at < 0 or projected.shape[1] < at + (q_heads + kv_heads) * maps * dim + kv_heads * vdim:
+        if keyed_values and (vdim != dim or maps != 1):
+            self._refuse("values that are the keys are as wide as they, one map a head")
+        if (projected.dim() != 2 or at < 0
+                or projected.shape[1] < at + (q_heads + kv_heads) * maps * dim + (0 if keyed_values else kv_heads * vdim)):
             self._refuse(f"projected rows must hold queries, keys and values, got {tuple(projected.shape)}")
         self._dense(q_out, "q_out", projected.dtype, (tokens, q_heads * maps * dim))
         num_pages, page_size = self._gated_pages(k_pages, v_pages, kv_heads, maps * dim, vdim, projected.dtype)
@@ -802,7 +857,8 @@ class PartsKernels:
             rot_dims if table is not None else 0,
             _ptr(positions) if table is not None or temperature is not None else ctypes.c_void_p(0),
             _ptr(q_weight), _ptr(k_weight), 1 if whole else 0, 1 if interleaved else 0,
-            ctypes.c_float(value_eps if value_eps is not None else -1.0), ctypes.c_float(coef), every, self._stream()),
+            ctypes.c_float(value_eps if value_eps is not None else -1.0), ctypes.c_float(coef), every,
+            1 if keyed_values else 0, self._stream()),
             "unit_norm_write")
 
     def gated_attention(self, q, k_pages, v_pages, gates, gate_at, ctx, meta, q_heads, kv_heads, dim, vdim, scale, softcap,

@@ -246,16 +246,33 @@ class ScaledDelta(Unsettled):
     """A branch's output that is added to the residual sum times a constant: stream += scale * delta - and then, where
     the model's pass has given one, a vector `offset` that every row takes (what a pass over repeated layers adds before
     its first layer).  `delta` None: the offset alone.  `second`: the output of a second branch that read the same
-    input - stream += scale * (delta + second), the two added in float32."""
+    input - stream += scale * (delta + second), the two added in float32.  `second` may be an `InputShare`: a branch's rows
+    and a share of what it read, which is added the same way."""
 
     def __init__(self, delta: torch.Tensor | None, scale: float, kernels, offset: torch.Tensor | None = None,
-                 second: torch.Tensor | None = None):
+                 second: "torch.Tensor | InputShare | None" = None):
         self.delta, self.scale, self.kernels, self.offset, self.second = delta, float(scale), kernels, offset, second
 
+    def extras(self) -> dict:
+        """What `norm_add_norm` is told beside the delta and its scale."""
+        if self.second is None:
+            return {"offset": self.offset}
+        if isinstance(self.second, InputShare):
+            return {"offset": self.offset, "delta2": self.second.delta, "share": self.second.rows,
+                    "share_weights": self.second.weights, "share_at": self.second.column}
+        return {"offset": self.offset, "delta2": self.second}
+
     def settle(self, stream: torch.Tensor) -> None:
-        more = {"delta2": self.second} if self.second is not None else {}
-        self.kernels.norm_add_norm(stream, self.delta, None, 0.0, None, 0.0, None, delta_scale=self.scale, offset=self.offset,
-                                   **more)
+        self.kernels.norm_add_norm(stream, self.delta, None, 0.0, None, 0.0, None, delta_scale=self.scale, **self.extras())
+
+
+class InputShare:
+    """The output of a branch that hands on a share of its own input beside what it computed: row t of it is
+    delta[t] + weights[t, column] * rows[t] (weights float32).  Returned by a feed-forward whose block has said that it takes
+    one (`ctx.takes_input_share`); the block adds both to the residual sum in one kernel."""
+
+    def __init__(self, delta: torch.Tensor, rows: torch.Tensor, weights: torch.Tensor, column: int):
+        self.delta, self.rows, self.weights, self.column = delta, rows, weights, int(column)
 
 
 class NormedDelta(Unsettled):

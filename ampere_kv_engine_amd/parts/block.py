@@ -233,7 +233,9 @@ class SharedNormBlock(Part):
         ctx.fold_into_stream, ctx.fold_gain = False, None      # no branch of this block adds itself to the stream
         normed = self.norm.after(stream, pending, ctx.arena.take((stream.shape[0], self.hidden), self.rt.dtype))
         mixed = self.mixer.forward(normed, ctx, cache, writes_cache)
+        ctx.takes_input_share = True            # (the next norm's kernel adds what the branch hands on of its input)
         other = self.feed_forward.forward(normed, ctx) if self.has_feed_forward else None
+        ctx.takes_input_share = False
         return ScaledDelta(mixed, self.scale, self.rt.kernels, second=other)
 
 

@@ -18,9 +18,12 @@
     with `value_norm_eps`: every head's value divided by its root mean square (no weight) before it is cached
     with `distance_bias`: score - r1_h ln(1 + r2_h (i - j)), after the softcap (tensors `r1`, `r2`, a number per head, kept
     float32)
+    with `values="keys"`: v = k as it was projected - before norm, rotation or anything else -, there is no W_v, and
+    value_dim is head_dim
+    with `out_bias_suffix`: the output product has a bias, named after its matrix with this suffix
 
 Keys are `head_dim` wide, values `value_dim`; query head h reads kv head h // (q_heads / kv_heads).  Keys are cached
-after their norm.  All five projections are one product over the layer's input.
+after their norm.  All projections are one product over the layer's input.
 """
 
 from __future__ import annotations
@@ -71,6 +74,11 @@ class GatedAttention(Part, SharesProducts):
         self.has_bias = bool(spec.get("distance_bias", False))
         self.distance_bias = None
         self.head_gate = bool(spec.get("head_gate", False))
+        if spec.get("values", "projected") not in ("projected", "keys"):
+            raise ValueError(f"values are 'projected' or the 'keys', not {spec['values']!r}")
+        self.keyed_values = spec.get("values") == "keys"
+        if self.keyed_values and self.vdim != self.dim:
+            raise ValueError(f"values that are the keys are as wide as they, not {self.vdim} beside {self.dim}")
         self.name = spec.get("name", "attn")
         if self.q_heads % self.kv_heads:
             raise ValueError(f"q_heads {self.q_heads} is not a multiple of kv_heads {self.kv_heads}")
@@ -79,12 +87,16 @@ class GatedAttention(Part, SharesProducts):
                 raise ValueError(f"{what} must be positive or None, got {value}")
         if self.softcap is not None and self.softcap <= 0:
             raise ValueError(f"softcap must be positive or None, got {self.softcap}")
-        self.q_size, self.k_size, self.v_size = self.q_heads * self.dim, self.kv_heads * self.dim, self.kv_heads * self.vdim
+        self.q_size, self.k_size = self.q_heads * self.dim, self.kv_heads * self.dim
+        self.v_size = 0 if self.keyed_values else self.kv_heads * self.vdim      # (columns of its own in the projection)
         names = dict(q="q", k="k", v="v", g="g", o="o", sink="sink", r1="r1", r2="r2")
         names.update(spec.get("names") or {})
         self.names = names
         bias = spec.get("bias_suffix")           # q, k and v have bias vectors named after them, with this suffix
-        sizes, stacked = [self.q_size, self.k_size, self.v_size], [names["q"], names["k"], names["v"]]
+        sizes, stacked = [self.q_size, self.k_size], [names["q"], names["k"]]
+        if not self.keyed_values:
+            sizes.append(self.v_size)
+            stacked.append(names["v"])
         biases = [n + bias for n in stacked] if bias else None
         if self.head_gate:
             sizes.append(self.q_heads)
@@ -93,9 +105,11 @@ class GatedAttention(Part, SharesProducts):
                 biases.append(None)
         self.width = sum(sizes)
         self.qkvg = self.inputs = Linear(runtime, self.hidden, sizes, stacked, bias_names=biases)
-        if self.learned_sink or self.has_bias:
+        out_bias = spec.get("out_bias_suffix")
+        self.out = self.outputs = Linear(runtime, self.q_heads * self.vdim, [self.hidden], [names["o"]],
+                                         bias_names=[names["o"] + out_bias] if out_bias else None)
+        if self.learned_sink or self.has_bias or out_bias:
             self.inputs = None      # (a tensor of its own beside the products: side by side with others it runs by itself)
-        self.out = self.outputs = Linear(runtime, self.q_heads * self.vdim, [self.hidden], [names["o"]])
         runtime.kernels.check_gated_attention_sizes(self.q_heads, self.kv_heads, self.dim, self.vdim, runtime.page_size)
 
     def _prefix(self, prefix):
@@ -152,6 +166,8 @@ class GatedAttention(Part, SharesProducts):
             rotation.update(q_weight=self.q_norm_weight, k_weight=self.k_norm_weight, whole=True)
         if self.value_eps is not None:
             rotation["value_eps"] = self.value_eps
+        if self.keyed_values:
+            rotation["keyed_values"] = True
         if self.temperature is not None:
             rotation.update(temperature=self.temperature, positions=ctx.positions)
         k.unit_norm_write(projected, self.q_heads, self.kv_heads, self.dim, self.vdim, eps,

@@ -86,9 +86,8 @@ class RMSNorm(Norm):
                                           delta_scale=pending.scale, delta2=pending.second, post_weight2=pending.second_weight)
             return out
         if isinstance(pending, ScaledDelta) and self.single_rounding:      # one kernel: add the branch times its constant, norm
-            more = {"delta2": pending.second} if pending.second is not None else {}
             self.rt.kernels.norm_add_norm(stream, pending.delta, None, 0.0, self.weight, self.eps, out,
-                                          delta_scale=pending.scale, offset=pending.offset, **more)
+                                          delta_scale=pending.scale, **pending.extras())
             return out
         if (pending is None or not isinstance(pending, NormedDelta)
                 or not (self.single_rounding and type(pending.norm) is RMSNorm and pending.norm.single_rounding)):

@@ -273,12 +273,15 @@ class TorchKernels(KernelSet):
         words[ctx.seq_slots.long(), 7] = cur[ctx.q_start.long()[1:] - 1].int()
 
     def norm_add_norm(self, stream, delta, post_weight, post_eps, pre_weight, pre_eps, out, delta_scale=1.0, offset=None,
-                      delta2=None, post_weight2=None):
+                      delta2=None, post_weight2=None, share=None, share_weights=None, share_at=0):
         if post_weight2 is not None:       # two branches, each normed by itself
             unit = lambda v: v * torch.rsqrt((v * v).mean(-1, keepdim=True) + post_eps)
             stream += delta_scale * (unit(delta.float()) * post_weight + unit(delta2.float()) * post_weight2)
         elif delta is not None:
-            d = (delta.float() + delta2.float() if delta2 is not None else delta.float()) * delta_scale
+            d = delta.float() + delta2.float() if delta2 is not None else delta.float()
+            if share is not None:              # a share of what a branch read, weighted row by row
+                d = d + share_weights[:, share_at, None] * share.float()
+            d = d * delta_scale
             if post_weight is not None:
                 d = d * torch.rsqrt((d * d).mean(-1, keepdim=True) + post_eps) * post_weight
             stream += d
@@ -286,6 +289,9 @@ class TorchKernels(KernelSet):
             stream += offset
         if out is not None:
             out.copy_((stream * torch.rsqrt((stream * stream).mean(-1, keepdim=True) + pre_eps) * pre_weight).to(out.dtype))
+
+    def add_weighted_rows(self, rows, weights, column, out):
+        out.copy_((out.float() + weights[:, column, None] * rows.float()).to(out.dtype))
 
     def embed_add(self, ids, table, out, ctx=None):
         """out[n] += table[id]; an id of -1 is the token chosen last for the row's request."""
@@ -541,13 +547,14 @@ class TorchKernels(KernelSet):
 
     def unit_norm_write(self, projected, q_heads, kv_heads, dim, vdim, eps, slot_map, k_pages, v_pages, q_out, at=0, maps=1,
                         table=None, rot_dims=0, positions=None, q_weight=None, k_weight=None, whole=False, interleaved=False,
-                        value_eps=None, temperature=None):
+                        value_eps=None, temperature=None, keyed_values=False):
         projected = projected[:, at:]
         n = projected.shape[0]
         q_size, k_size, v_size = q_heads * maps * dim, kv_heads * maps * dim, kv_heads * vdim
         q = projected[:, :q_size].reshape(n, q_heads * maps, dim).float()
         k = projected[:, q_size:q_size + k_size].reshape(n, kv_heads * maps, dim).float()
-        v = projected[:, q_size + k_size:q_size + k_size + v_size].reshape(n, kv_heads, vdim)
+        v_at = q_size if keyed_values else q_size + k_size      # (values that are the keys, as they were projected)
+        v = projected[:, v_at:v_at + v_size].reshape(n, kv_heads, vdim)
         if eps is not None:
             over = (-2, -1) if whole else -1        # (`whole`: one root mean square for all of a token's query vectors)
             q = q * torch.rsqrt((q * q).mean(over, keepdim=True) + eps)
@@ -683,6 +690,17 @@ class TorchKernels(KernelSet):
         if logits.shape[1] > experts:
             gates[:, experts:] = torch.sigmoid(logits[:, experts:])
 
+    def route_corrected(self, logits, correction, gates, experts, top, shared):
+        scores = logits.softmax(-1)
+        chosen = torch.sort(scores + correction, dim=-1, descending=True, stable=True).indices[:, :top]
+        picked = torch.gather(scores, 1, chosen)
+        weights = torch.zeros_like(scores).scatter_(1, chosen, picked / (picked.sum(-1, keepdim=True) + 1e-20))
+        gates[:, :experts] = weights[:, :experts]
+        if shared:
+            gates[:, experts] = 1.0
+        if logits.shape[1] > experts:
+            gates[:, -1] = weights[:, experts:].sum(-1)
+
     def gate_activation(self, up, gates, act, experts, ff, activation, inside):
         columns = act.shape[1]
         weight = gates[:, :experts].repeat_interleave(ff, dim=1)
@@ -697,12 +715,19 @@ class TorchKernels(KernelSet):
         act.copy_(torch.where(weight != 0, value, torch.zeros_like(value)).to(act.dtype))
 
     def gate_silu_mul(self, gate_up, gates, act, experts, ff):
+        inf = float("inf")
+        self.gate_clamped_mul(gate_up, gates, act, experts, ff, inf, 1.0, 0.0, inf)
+
+    def gate_clamped_mul(self, gate_up, gates, act, experts, ff, limit, slope, shift, shared_limit):
         columns = act.shape[1]
         g, u = gate_up[:, :columns].float(), gate_up[:, columns:].float()
+        bound = torch.full((columns,), limit)
+        bound[experts * ff:] = shared_limit
+        g, u = torch.minimum(g, bound), torch.maximum(torch.minimum(u, bound), -bound)
         weight = gates[:, :experts].repeat_interleave(ff, dim=1)
         if columns > experts * ff:
             weight = torch.cat((weight, gates[:, experts:experts + 1].expand(-1, columns - experts * ff)), dim=1)
-        act.copy_((weight * (g * torch.sigmoid(g) * u)).to(act.dtype))
+        act.copy_((weight * (g * torch.sigmoid(slope * g) * (u + shift))).to(act.dtype))
 
     # ---- sampling -----------------------------------------------------------------------------------------
     def sample(self, logits, temperature, seeds, draws, out):
