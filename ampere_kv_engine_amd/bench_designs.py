@@ -1,4 +1,4 @@
-"""Prefill and decode throughput of the Keranex design (and, `--workload tukevik` / `lirulix` / `mekuvik` / `bolatar`, of those designs) at sizes that resemble a real model's layers (random weights),
+"""Prefill and decode throughput of the Keranex design (and, `--workload tukevik` / `lirulix` / `mekuvik` / `bolatar` / `ziferax`, of those designs) at sizes that resemble a real model's layers (random weights),
 beside the dense Qwen3 decoder at equal width, depth, heads and active feed-forward width - the closest model the
 engine has.  `python bench.py --workload keranex [--design-sizes s,m] [--layers L]` prints one JSON line per size:
 
@@ -170,6 +170,37 @@ def bolatar_config(size: dict, layers: int) -> dict:
                 layers=[dict(type=kind, mixer=mixer, mlp=mlp) for kind, mixer in (pattern[i % 4] for i in range(layers))])
 
 
+# Ziferax at the same widths: every layer attention over a window with values that are the keys, and routed experts with a
+# shared one and identity experts (a token chooses `top` of experts + identity); every fourth layer runs the tensors of the
+# one three before it.  Beside it Mekuvik with the same width, depth, heads, window and experts (the closest design the engine
+# has: one norm a layer, the same attention kernels, routed experts with a shared one; its experts have no gate) and Qwen3 with
+# a feed-forward as wide as the experts a token uses.
+ZIFERAX_SIZES = {
+    "s": dict(width=2048, vocab=32768, heads=16, kv_heads=4, dim=128, vdim=128, rot=64, window=1024, experts=16, identity=4, top=3,
+              ff=1024, shared=1024, dense=3072),
+    "m": dict(width=4096, vocab=65536, heads=32, kv_heads=8, dim=128, vdim=128, rot=64, window=2048, experts=32, identity=8, top=5,
+              ff=1024, shared=1024, dense=5120),
+}
+
+
+def ziferax_config(size: dict, layers: int) -> dict:
+    mixer = dict(heads=size["heads"], kv_heads=size["kv_heads"], dim=size["dim"], vdim=size["vdim"], scale=size["dim"] ** -0.5,
+                 rot=dict(dims=size["rot"], base=1e6), mask=dict(size=size["window"]))
+    mlp = dict(kind="moe", expert=dict(ff=size["ff"], limit=7.0), shared=dict(ff=size["shared"], limit=7.0),
+               router=dict(experts=size["experts"], identity=size["identity"], top=size["top"]))
+    return dict(architecture="Ziferax", vocab=size["vocab"], width=size["width"], norm=dict(eps=1e-6), residual_mult=0.5,
+                layers=[dict(type="attention", mixer=mixer, mlp=mlp, **({"weights_of": i - 3} if i % 4 == 3 else {})) for i in range(layers)])
+
+
+def mekuvik_beside_ziferax(size: dict, layers: int) -> dict:
+    window = dict(heads=size["heads"], kv_heads=size["kv_heads"], dim=size["dim"], vdim=size["vdim"], scale=size["dim"] ** -0.5,
+                  rot=dict(dims=size["rot"], base=1e6), mask=dict(size=size["window"], keep_first=4))
+    routed = dict(kind="moe", expert=dict(ff=size["ff"]), router=dict(experts=size["experts"], top=size["top"] - 1),
+                  shared=dict(ff=size["shared"]))
+    return dict(architecture="Mekuvik", vocab=size["vocab"], width=size["width"], norm=dict(eps=1e-6), logit_scale=0.5,
+                layers=[dict(type="attention", mixer=window, mlp=routed) for _ in range(layers)])
+
+
 def qwen3_beside_tukevik(size: dict, layers: int) -> dict:
     return dict(architectures=["Qwen3ForCausalLM"], num_hidden_layers=layers, hidden_size=size["width"],
                 num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=size["dim"],
@@ -234,76 +265,50 @@ def measure(config, batch: int, context: int, steps: int, warmup: int, graphs: b
     return out
 
 
+def _designs() -> dict:
+    """Per workload: its sizes, and what is measured at each - (name on the command line, key of the printed line,
+    configuration from (the size's name, layers))."""
+    from .config import BolatarConfig, KeranexConfig, LirulixConfig, MekuvikConfig, Qwen3Config, TukevikConfig, ZiferaxConfig
+    qwen3 = lambda sizes, width: (lambda name, n: Qwen3Config.from_dict(
+        qwen3_beside_tukevik(dict(sizes[name], dense=width(sizes[name])), n)))
+    dense, ff = (lambda size: size["dense"]), (lambda size: size["ff"])
+    return {
+        "keranex": (SIZES, (
+            ("keranex", "keranex", lambda name, n: KeranexConfig.from_dict(keranex_config(SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", lambda name, n: Qwen3Config.from_dict(qwen3_config(SIZES[name], n))))),
+        "tukevik": (TUKEVIK_SIZES, (
+            ("tukevik", "tukevik", lambda name, n: TukevikConfig.from_dict(tukevik_config(TUKEVIK_SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", qwen3(TUKEVIK_SIZES, dense)))),
+        "lirulix": (LIRULIX_SIZES, (
+            ("lirulix", "lirulix", lambda name, n: LirulixConfig.from_dict(lirulix_config(LIRULIX_SIZES[name], n))),
+            ("tukevik", "tukevik_equal_size", lambda name, n: TukevikConfig.from_dict(tukevik_beside_lirulix(LIRULIX_SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", qwen3(LIRULIX_SIZES, ff)))),
+        "mekuvik": (MEKUVIK_SIZES, (
+            ("mekuvik", "mekuvik", lambda name, n: MekuvikConfig.from_dict(mekuvik_config(MEKUVIK_SIZES[name], n))),
+            ("tukevik", "tukevik_equal_size", lambda name, n: TukevikConfig.from_dict(tukevik_config(TUKEVIK_SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", qwen3(TUKEVIK_SIZES, dense)))),
+        "bolatar": (BOLATAR_SIZES, (
+            ("bolatar", "bolatar", lambda name, n: BolatarConfig.from_dict(bolatar_config(BOLATAR_SIZES[name], n))),
+            ("lirulix", "lirulix_equal_size", lambda name, n: LirulixConfig.from_dict(lirulix_config(LIRULIX_SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", qwen3(LIRULIX_SIZES, ff)))),
+        "ziferax": (ZIFERAX_SIZES, (
+            ("ziferax", "ziferax", lambda name, n: ZiferaxConfig.from_dict(ziferax_config(ZIFERAX_SIZES[name], n))),
+            ("mekuvik", "mekuvik_equal_size", lambda name, n: MekuvikConfig.from_dict(mekuvik_beside_ziferax(ZIFERAX_SIZES[name], n))),
+            ("qwen3", "qwen3_equal_size", qwen3(ZIFERAX_SIZES, dense)))),
+    }
+
+
 def design_workload(sizes: str, layers: int | None, batch: int, context: int, steps: int, warmup: int,
                     graphs: bool = True, only: str = "", design: str = "keranex") -> int:
-    from .config import BolatarConfig, KeranexConfig, LirulixConfig, MekuvikConfig, Qwen3Config, TukevikConfig
-    for name in [s for s in sizes.split(",") if s and design == "bolatar"]:
-        size, beside = BOLATAR_SIZES[name], LIRULIX_SIZES[name]
-        count = layers or 8
-        line = {"workload": "bolatar", "sizes": name, "layers": count, "batch": batch, "context": context,
-                "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
-                "shape": size}
-        if only in ("", "bolatar"):
-            line["bolatar"] = measure(BolatarConfig.from_dict(bolatar_config(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "lirulix"):
-            line["lirulix_equal_size"] = measure(LirulixConfig.from_dict(lirulix_config(beside, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "qwen3"):
-            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_beside_tukevik(dict(beside, dense=beside["ff"]), count)), batch, context, steps, warmup, graphs)
-        print(json.dumps(line), flush=True)
-    if design == "bolatar":
-        return 0
-    for name in [s for s in sizes.split(",") if s and design == "mekuvik"]:
-        size, beside = MEKUVIK_SIZES[name], TUKEVIK_SIZES[name]
-        count = layers or 8
-        line = {"workload": "mekuvik", "sizes": name, "layers": count, "batch": batch, "context": context,
-                "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
-                "shape": size}
-        if only in ("", "mekuvik"):
-            line["mekuvik"] = measure(MekuvikConfig.from_dict(mekuvik_config(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "tukevik"):
-            line["tukevik_equal_size"] = measure(TukevikConfig.from_dict(tukevik_config(beside, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "qwen3"):
-            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_beside_tukevik(beside, count)), batch, context, steps, warmup, graphs)
-        print(json.dumps(line), flush=True)
-    if design == "mekuvik":
-        return 0
-    for name in [s for s in sizes.split(",") if s and design == "lirulix"]:
-        size = LIRULIX_SIZES[name]
-        count = layers or 8
-        line = {"workload": "lirulix", "sizes": name, "layers": count, "batch": batch, "context": context,
-                "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
-                "shape": size}
-        if only in ("", "lirulix"):
-            line["lirulix"] = measure(LirulixConfig.from_dict(lirulix_config(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "tukevik"):
-            line["tukevik_equal_size"] = measure(TukevikConfig.from_dict(tukevik_beside_lirulix(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "qwen3"):
-            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_beside_tukevik(dict(size, dense=size["ff"]), count)), batch, context, steps, warmup, graphs)
-        print(json.dumps(line), flush=True)
-    if design == "lirulix":
-        return 0
-    for name in [s for s in sizes.split(",") if s and design == "tukevik"]:
-        size = TUKEVIK_SIZES[name]
-        count = layers or 8
-        line = {"workload": "tukevik", "sizes": name, "layers": count, "batch": batch, "context": context,
-                "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
-                "shape": size}
-        if only in ("", "tukevik"):
-            line["tukevik"] = measure(TukevikConfig.from_dict(tukevik_config(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "qwen3"):
-            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_beside_tukevik(size, count)), batch, context, steps, warmup, graphs)
-        print(json.dumps(line), flush=True)
-    if design == "tukevik":
-        return 0
+    known, models = _designs()[design]
     for name in [s for s in sizes.split(",") if s]:
-        size = SIZES[name]
+        size = known[name]
         count = layers or 8
-        line = {"workload": "keranex", "sizes": name, "layers": count, "batch": batch, "context": context,
+        line = {"workload": design, "sizes": name, "layers": count, "batch": batch, "context": context,
                 "prefill_tokens": PREFILL_TOKENS, "dtype": "bf16", "data": "synthetic: random-init weights, random token ids",
                 "shape": size}
-        if only in ("", "keranex"):
-            line["keranex"] = measure(KeranexConfig.from_dict(keranex_config(size, count)), batch, context, steps, warmup, graphs)
-        if only in ("", "qwen3"):
-            line["qwen3_equal_size"] = measure(Qwen3Config.from_dict(qwen3_config(size, count)), batch, context, steps, warmup, graphs)
+        for model, key, config in models:
+            if only in ("", model):
+                line[key] = measure(config(name, count), batch, context, steps, warmup, graphs)
         print(json.dumps(line), flush=True)
     return 0

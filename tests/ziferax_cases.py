@@ -48,20 +48,22 @@ ZIFERAX_C = dict(
 ZIFERAX = {"A": (ZIFERAX_A, 101, 4), "B": (ZIFERAX_B, 102, 8), "C": (ZIFERAX_C, 103, 16)}        # config, weight seed, page size
 
 LENGTHS, PROMPTS, POOL_TOKENS = K.LENGTHS, K.PROMPTS, K.POOL_TOKENS
-# float32: a few hundred float32 operations a position.  bfloat16: as served, against the plain float32 logits; a tenth of a
-# request's positions may lie beyond, where a rounded activation turns a router's close call.
-LIMITS = {"float32": dict(max=2e-4, rms=2e-4), "bfloat16": dict(max=0.08, rms=0.1)}
+# float32: a few hundred float32 operations a position.  bfloat16: as served, against the plain float32 logits: positions lie
+# within 0.02 (median 0.004 to 0.01); a tenth of a request's positions may lie beyond, where a rounded activation turns a
+# router's close call.
+LIMITS = {"float32": dict(max=2e-4, rms=2e-4), "bfloat16": dict(max=0.045, rms=0.055)}
 BEYOND = {"float32": 0.0, "bfloat16": 0.1}
 
 
 def sharpen(folder: str, raw: dict, seed: int = 0) -> None:
     """Random tensors of N(0, 0.02) hide faults: softmaxes are flat and one key more or less hardly shows, a sink is one key
     among many, biases vanish, nothing reaches a limit, the router's scores are all alike and its corrections change no
-    choice.  Projections, biases, routers and experts are scaled; sinks and corrections are drawn over the range in which
-    they matter."""
+    choice.  Projections, biases, routers and experts are scaled - to the same effect at any width -; sinks and corrections
+    are drawn over the range in which they matter."""
     path = os.path.join(folder, "model.safetensors")
     tensors = load_file(path)
     generator = torch.Generator().manual_seed(9100 + seed)
+    by_width = (88.0 / raw["width"]) ** 0.5
 
     def scale(name, factor):
         tensors[name] = (tensors[name].float() * factor).to(torch.bfloat16)
@@ -72,19 +74,21 @@ def sharpen(folder: str, raw: dict, seed: int = 0) -> None:
     scale("embed", 25.0)
     for name in list(tensors):
         if name.endswith((".mix.q", ".mix.k")):
-            scale(name, 15.0)
+            scale(name, 9.0 * by_width)
         elif name.endswith((".mix.q.b", ".mix.k.b", ".mix.o.b")):
             scale(name, 20.0)
         elif name.endswith(".mix.o"):
-            scale(name, 4.0)
+            scale(name, 6.0)
         elif name.endswith(".mix.sink"):
             uniform(name, -1.0, 4.0)
         elif name.endswith(".mlp.router"):
-            scale(name, 12.0)
+            scale(name, 12.0 * by_width)
         elif name.endswith(".mlp.correction"):
             uniform(name, -0.3, 0.3)
+        elif ".mlp." in name and not name.endswith(".down"):
+            scale(name, 7.0 * by_width)
         elif ".mlp." in name:
-            scale(name, 8.0)
+            scale(name, 7.0)
     save_file(tensors, path, metadata={"format": "pt"})
 
 
@@ -150,6 +154,17 @@ def check(engine, case, schedule):
     return pages
 
 
+def check_spread(engine, case, schedule) -> None:
+    """For drawn configurations as they are served: many experts and layers make many close calls, so not every position is
+    held to the limit - the middle one is, and three quarters of them to twice that."""
+    got, _ = schedules.run(engine, case["requests"], schedule)
+    errors = torch.cat([(got[name] - want).abs().amax(1) / want.abs().max() for name, want in case["expected"].items()])
+    assert not torch.isnan(errors).any(), "NaN logits"
+    median, most, limit = float(errors.median()), float(errors.quantile(0.75)), LIMITS[engine.config.dtype]["max"]
+    assert median < limit and most < 2 * limit, f"{case['name']}: median {median:.4f}, three quarters within {most:.4f}"
+    print(f"[ziferax {case['name']} {engine.config.dtype}] median error {median:.4f}, three quarters within {most:.4f}")
+
+
 # ---- the cuttings (those of the other designs' cases, held to this design's limits) -----------------------------------
 
 def _with_this_check(cutting):
@@ -182,14 +197,14 @@ CUTTINGS = [case_whole, case_prefill_then_token_by_token, case_token_by_token_fr
 
 def alone(mechanism: str) -> tuple:
     """(config, weight seed, page size) of a small model in which one mechanism alone shapes the logits."""
-    tiny, plain_attention = ATTN(1, 1, 8, 0.3, 2, 4, 100.0), ATTN(4, 2, 16, 0.35)
+    tiny, plain_attention, calm = ATTN(1, 1, 8, 0.3, 2, 4, 100.0), ATTN(4, 2, 16, 0.35), ATTN(4, 2, 16, 0.15, None, 8, 100.0)
     layers = {
         "windowed attention": [LAYER(ATTN(4, 2, 16, 0.35, 11, 12, 1000.0), None)],
         "attention without rotation or window": [LAYER(plain_attention, None)],
         "experts chosen by corrected scores": [LAYER(tiny, MOE(9, 0, 3, 12, 5.0))],
         "identity experts": [LAYER(tiny, MOE(2, 7, 4, 8, 5.0))],
         "shared expert": [LAYER(tiny, MOE(1, 0, 1, 8, 0.4, 36, 0.8))],
-        "tensors run again": [LAYER(plain_attention, None), LAYER(tiny, MOE(3, 1, 2, 8, 1.0)), LAYER(plain_attention, None, 0), LAYER(plain_attention, None, 0)],
+        "tensors run again": [LAYER(calm, None), LAYER(tiny, MOE(3, 1, 4, 8, 1.0)), LAYER(calm, None, 0), LAYER(calm, None, 0)],
     }
     raw = dict(architecture="Ziferax", vocab=150, width=48, norm=dict(eps=1e-6), residual_mult=0.8, layers=layers[mechanism])
     return raw, 111 + sorted(layers).index(mechanism), 4
