@@ -143,6 +143,8 @@ class Part:
         that product norms the rows itself where the kernel set can (`UnnormedRows.product`), else the rows are
         normed first (`UnnormedRows.rows`).  A norm offers them through `Norm.pending` / `Norm.scaled`, which return
         None for a norm that can only be computed at once.
+      * `InputShare` - a feed-forward's output beside a share of the rows it read, returned only while the block has
+        `ctx.takes_input_share` set: the block's `ScaledDelta` carries it to the kernel of the next norm.
       * nothing else: a part without these flags gets and returns tensors `[tokens, width]` in `runtime.dtype`.
 
     The kernel set's side of the protocol is `KernelSet` below: capabilities that default to "no".
